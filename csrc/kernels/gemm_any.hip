@@ -51,6 +51,8 @@ __device__ __forceinline__ float epi_val(const AnyGemmArgs& p, float g, float u)
   }
   if (p.act == 3) return tanhf(g);
   if (p.act == 4) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
+  if (p.act == 5) return 0.5f * g * (1.f + erff(g * 0.70710678118654752f));
+  if (p.act == 6) { const float r = fmaxf(g, 0.f); return r * r; }
   return g;
 }
 

@@ -1,6 +1,7 @@
 // Row-wise kernels of layered hybrid models over an fp32 residual stream: embedding gather into
-// fp32, RMS norm with a scalar or vector weight (fp32 statistics, bf16 or fp32 rows in and out,
+// fp32, RMS or layer norm with a scalar or vector weight (fp32 statistics, bf16 or fp32 rows in and out,
 // optional row gather), a tanh norm without statistics, the gated residual update of a parallel layer,
+// the residual update of pre-norm and sandwich-norm layers with the next sublayer's norm,
 // the read / write of a sublayer over several learned-weight copies of the stream, and mixture-of-experts
 // routing (sigmoid or softmax scores with an optional selection-only correction, top-k, counting sort by
 // expert, weighted combine with an optional shared-expert row). Every kernel reads its sizes from arguments and its per-step metadata from device
@@ -22,36 +23,42 @@ __device__ __forceinline__ float sigm(float x) { return 1.f / (1.f + expf(-x)); 
 
 __global__ __launch_bounds__(256) void norm_rows_kernel(const void* __restrict__ x, int64_t ldx_, int x_f32,
                                                          const int32_t* __restrict__ rows,
-                                                         const float* __restrict__ w, int w_scalar, float eps,
+                                                         const float* __restrict__ w, int w_scalar, float eps, int center,
                                                          void* __restrict__ y, int64_t ldy, int y_f32, int n) {
   __shared__ float red[16];
   const int m = blockIdx.x;
   const int64_t src = rows ? rows[m] : m;
   const int64_t xo = src * ldx_;
+  float mean = 0.f;
+  if (center) {  // (uniform)
+    float s = 0.f;
+    for (int c = threadIdx.x; c < n; c += blockDim.x) s += ldx(x, xo + c, x_f32);
+    mean = block_reduce_sum(s, red) / (float)n;
+  }
   float ss = 0.f;
   for (int c = threadIdx.x; c < n; c += blockDim.x) {
-    const float v = ldx(x, xo + c, x_f32);
+    const float v = ldx(x, xo + c, x_f32) - mean;
     ss = fmaf(v, v, ss);
   }
   ss = block_reduce_sum(ss, red);
   const float inv = 1.f / sqrtf(ss / (float)n + eps);
   const float ws = w_scalar ? w[0] : 1.f;
   for (int c = threadIdx.x; c < n; c += blockDim.x) {
-    const float v = ldx(x, xo + c, x_f32) * inv * (w_scalar ? ws : w[c]);
+    const float v = (ldx(x, xo + c, x_f32) - mean) * inv * (w_scalar ? ws : w[c]);
     stx(y, (int64_t)m * ldy + c, y_f32, v);
   }
 }
 
 __global__ __launch_bounds__(256) void embed_rows_kernel(const int32_t* __restrict__ ids,
                                                           const int32_t* __restrict__ prev,
-                                                          const void* __restrict__ table, int t_f32,
+                                                          const void* __restrict__ table, int t_f32, float scale,
                                                           float* __restrict__ x, int W, int vocab) {
   const int t = blockIdx.x;
   int tok = ids[t];
   if (tok < 0 && prev != nullptr) tok = prev[-tok - 1];
   const bool ok = tok >= 0 && tok < vocab;
   for (int c = threadIdx.x; c < W; c += blockDim.x)
-    x[(int64_t)t * W + c] = ok ? ldx(table, (int64_t)tok * W + c, t_f32) : 0.f;
+    x[(int64_t)t * W + c] = ok ? ldx(table, (int64_t)tok * W + c, t_f32) * scale : 0.f;
 }
 
 __global__ __launch_bounds__(256) void gated_residual_kernel(float* __restrict__ x, const void* __restrict__ y1,
@@ -101,6 +108,25 @@ __global__ __launch_bounds__(256) void glu_rows_kernel(const bf16_t* __restrict_
     }
     const float a = act == 4 ? 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x))) : x * sigm(x);
     g[e] = a * u[e];
+  }
+  *reinterpret_cast<uint4*>(out + t * ldo + j) = pack8(g);
+}
+
+// out[t][j] = act(x[t][j]), 8 columns per thread (every element is read and written by the same thread)
+__global__ __launch_bounds__(256) void act_rows_kernel(const bf16_t* x, int64_t ldx_, bf16_t* out, int64_t ldo, int n,
+                                                        int act, int64_t total) {
+  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= total) return;
+  const int per = n / 8;
+  const int64_t t = i / per;
+  const int j = (int)(i % per) * 8;
+  float g[8];
+  unpack8(ld16(x + t * ldx_ + j), g);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    if (act == 5) g[e] = 0.5f * g[e] * (1.f + erff(g[e] * 0.70710678118654752f));
+    else if (act == 6) { g[e] = fmaxf(g[e], 0.f); g[e] *= g[e]; }
+    else g[e] = tanhf(g[e]);
   }
   *reinterpret_cast<uint4*>(out + t * ldo + j) = pack8(g);
 }
@@ -194,7 +220,7 @@ __global__ __launch_bounds__(256) void hyper_mix_kernel(HyperArgs a) {
 // a wave-wide arg-max over the corrected scores (lowest index wins a tie)
 constexpr int RPL = 8;
 __global__ __launch_bounds__(256) void moe_route_wave_kernel(const float* __restrict__ z, const float* __restrict__ corr,
-                                                             int T, int E, int top, float norm_eps, int softmax, float scale,
+                                                             int T, int E, int top, float norm_eps, int score, float scale,
                                                              int32_t* __restrict__ idx, float* __restrict__ wts) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= T) return;  // (wave-uniform)
@@ -208,8 +234,8 @@ __global__ __launch_bounds__(256) void moe_route_wave_kernel(const float* __rest
     zmax = fmaxf(zmax, s[j]);
   }
   float den = 1.f;
-  if (softmax) {  // scores over all experts: exp(z - max) / sum
-    zmax = wave_reduce_max(zmax);
+  if (score != 0) zmax = wave_reduce_max(zmax);
+  if (score == 1) {  // scores over all experts: exp(z - max) / sum
     float part = 0.f;
 #pragma unroll
     for (int j = 0; j < RPL; ++j) part += lane + 64 * j < E ? expf(s[j] - zmax) : 0.f;
@@ -218,8 +244,9 @@ __global__ __launch_bounds__(256) void moe_route_wave_kernel(const float* __rest
 #pragma unroll
   for (int j = 0; j < RPL; ++j) {
     const int e = lane + 64 * j;
-    s[j] = softmax ? expf(s[j] - zmax) / den : sigm(s[j]);
-    v[j] = e < E ? s[j] + (corr ? corr[e] : 0.f) : -INFINITY;
+    const float z = s[j];
+    s[j] = score != 0 ? expf(z - zmax) / den : sigm(z);   // (score 2: den = 1, only the chosen ones' sum divides)
+    v[j] = e < E ? (score == 2 ? z : s[j]) + (corr ? corr[e] : 0.f) : -INFINITY;
   }
   float sum = 0.f, mine = 0.f;
   for (int c = 0; c < top; ++c) {
@@ -246,14 +273,15 @@ __global__ __launch_bounds__(256) void moe_route_wave_kernel(const float* __rest
 
 // one thread per token: `top` rounds of arg-max over the corrected scores (lowest index wins a tie)
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, const float* __restrict__ corr,
-                                                        int T, int E, int top, float norm_eps, int softmax, float scale,
+                                                        int T, int E, int top, float norm_eps, int score, float scale,
                                                         int32_t* __restrict__ idx, float* __restrict__ wts) {
   const int t = blockIdx.x * blockDim.x + threadIdx.x;
   if (t >= T) return;
   const float* zr = z + (int64_t)t * E;
   float zmax = -INFINITY, den = 1.f;
-  if (softmax) {  // scores over all experts: exp(z - max) / sum
+  if (score != 0)
     for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, zr[e]);
+  if (score == 1) {  // scores over all experts: exp(z - max) / sum
     den = 0.f;
     for (int e = 0; e < E; ++e) den += expf(zr[e] - zmax);
   }
@@ -265,8 +293,8 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
       bool taken = false;
       for (int d = 0; d < c; ++d) taken |= idx[(int64_t)t * top + d] == e;
       if (taken) continue;
-      const float s = softmax ? expf(zr[e] - zmax) / den : sigm(zr[e]);
-      const float v = s + (corr ? corr[e] : 0.f);
+      const float s = score != 0 ? expf(zr[e] - zmax) / den : sigm(zr[e]);
+      const float v = (score == 2 ? zr[e] : s) + (corr ? corr[e] : 0.f);
       if (best < 0 || v > bv) { best = e; bv = v; bs = s; }
     }
     idx[(int64_t)t * top + c] = best;
@@ -304,41 +332,89 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int32_t* __restric
   }
 }
 
-// x[t] += mult * y[t] (fp32 sum); with w: h[t] = x[t] / sqrt(mean(x[t]^2) + eps) * w from the new row. One workgroup
-// per token; the row stays in registers between the add and the norm (W <= 256 * RN_MAX), else it is read again.
+// x[t] += mult * u[t] (fp32 sum); with w: h[t] = norm(x[t]) * w from the new row. u[t]: the row of y, with GATHER the
+// weighted sum of the token's expert rows (choices ascending), with POST normed and weighted by post_w. CENTER: layer
+// norms. One workgroup per token; the row stays in registers between the norms and the add (W <= 256 * RN_MAX), the
+// columns beyond are read again.
 constexpr int RN_MAX = 16;
-__global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ x, const void* __restrict__ y, int y_f32,
-                                                             float mult, const float* __restrict__ w, float eps,
-                                                             void* __restrict__ h, int h_f32, int W) {
+template <bool POST, bool CENTER, bool GATHER>
+__global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) {
   __shared__ float red[16];
-  const int t = blockIdx.x;
-  float* xr = x + (int64_t)t * W;
+  const int t = blockIdx.x, W = a.W, tid = threadIdx.x;
+  float* xr = a.x + (int64_t)t * W;
+  const float fw = (float)W;
+  auto row = [&](int c) {
+    if (!GATHER) return ldx(a.y, (int64_t)t * W + c, a.y_f32);
+    float u = 0.f;
+    for (int k = 0; k < a.top; ++k)
+      u = fmaf(a.wts[(int64_t)t * a.top + k], ldx(a.y, (int64_t)a.pos[(int64_t)t * a.top + k] * W + c, a.y_f32), u);
+    return u;
+  };
   float keep[RN_MAX];
-  float ss = 0.f;
+  float pmean = 0.f, pinv = 1.f;
+  if (POST) {
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < RN_MAX; ++i) {
+      const int c = tid + 256 * i;
+      if (c < W) {
+        keep[i] = row(c);
+        s = CENTER ? s + keep[i] : fmaf(keep[i], keep[i], s);
+      }
+    }
+    for (int c = tid + 256 * RN_MAX; c < W; c += 256) {
+      const float u = row(c);
+      s = CENTER ? s + u : fmaf(u, u, s);
+    }
+    s = block_reduce_sum(s, red);
+    if (CENTER) {
+      pmean = s / fw;
+      s = 0.f;
+#pragma unroll
+      for (int i = 0; i < RN_MAX; ++i)
+        if (tid + 256 * i < W) { const float d = keep[i] - pmean; s = fmaf(d, d, s); }
+      for (int c = tid + 256 * RN_MAX; c < W; c += 256) { const float d = row(c) - pmean; s = fmaf(d, d, s); }
+      s = block_reduce_sum(s, red);
+    }
+    pinv = 1.f / sqrtf(s / fw + a.eps);
+  }
+  float s = 0.f;
 #pragma unroll
   for (int i = 0; i < RN_MAX; ++i) {
-    const int c = threadIdx.x + 256 * i;
+    const int c = tid + 256 * i;
     if (c < W) {
-      const float v = fmaf(mult, ldx(y, (int64_t)t * W + c, y_f32), xr[c]);
+      const float u = POST ? (keep[i] - pmean) * pinv * a.post_w[c] : row(c);
+      const float v = fmaf(a.mult, u, xr[c]);
       xr[c] = v;
       keep[i] = v;
-      ss = fmaf(v, v, ss);
+      s = CENTER ? s + v : fmaf(v, v, s);
     }
   }
-  for (int c = threadIdx.x + 256 * RN_MAX; c < W; c += 256) {
-    const float v = fmaf(mult, ldx(y, (int64_t)t * W + c, y_f32), xr[c]);
+  for (int c = tid + 256 * RN_MAX; c < W; c += 256) {
+    const float u = POST ? (row(c) - pmean) * pinv * a.post_w[c] : row(c);
+    const float v = fmaf(a.mult, u, xr[c]);
     xr[c] = v;
-    ss = fmaf(v, v, ss);
+    s = CENTER ? s + v : fmaf(v, v, s);
   }
-  if (w == nullptr) return;  // (uniform)
-  ss = block_reduce_sum(ss, red);
-  const float inv = 1.f / sqrtf(ss / (float)W + eps);
+  if (a.w == nullptr) return;  // (uniform)
+  s = block_reduce_sum(s, red);
+  float mean = 0.f;
+  if (CENTER) {
+    mean = s / fw;
+    s = 0.f;
+#pragma unroll
+    for (int i = 0; i < RN_MAX; ++i)
+      if (tid + 256 * i < W) { const float d = keep[i] - mean; s = fmaf(d, d, s); }
+    for (int c = tid + 256 * RN_MAX; c < W; c += 256) { const float d = xr[c] - mean; s = fmaf(d, d, s); }
+    s = block_reduce_sum(s, red);
+  }
+  const float inv = 1.f / sqrtf(s / fw + a.eps);
 #pragma unroll
   for (int i = 0; i < RN_MAX; ++i) {
-    const int c = threadIdx.x + 256 * i;
-    if (c < W) stx(h, (int64_t)t * W + c, h_f32, keep[i] * inv * w[c]);
+    const int c = tid + 256 * i;
+    if (c < W) stx(a.h, (int64_t)t * W + c, a.h_f32, (keep[i] - mean) * inv * a.w[c]);
   }
-  for (int c = threadIdx.x + 256 * RN_MAX; c < W; c += 256) stx(h, (int64_t)t * W + c, h_f32, xr[c] * inv * w[c]);
+  for (int c = tid + 256 * RN_MAX; c < W; c += 256) stx(a.h, (int64_t)t * W + c, a.h_f32, (xr[c] - mean) * inv * a.w[c]);
 }
 
 // out[t] = [a[t], b[t]] in out's dtype
@@ -442,10 +518,27 @@ void launch_glu_rows(const void* gu, int64_t ldg, void* out, int64_t ldo, int T,
                      reinterpret_cast<const bf16_t*>(gu), ldg, reinterpret_cast<bf16_t*>(out), ldo, n, act, limit, alpha, total);
 }
 
-void launch_residual_norm(float* x, const void* y, int y_f32, float mult, const float* w, float eps, void* h, int h_f32,
-                          int T, int W, hipStream_t st) {
-  if (T <= 0 || W <= 0) return;
-  hipLaunchKernelGGL(residual_norm_kernel, dim3(T), dim3(256), 0, st, x, y, y_f32, mult, w, eps, h, h_f32, W);
+void launch_act_rows(const void* x, int64_t ldx_, void* out, int64_t ldo, int T, int n, int act, hipStream_t st) {
+  const int64_t total = (int64_t)T * (n / 8);
+  if (total <= 0) return;
+  hipLaunchKernelGGL(act_rows_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, st,
+                     reinterpret_cast<const bf16_t*>(x), ldx_, reinterpret_cast<bf16_t*>(out), ldo, n, act, total);
+}
+
+template <bool POST, bool CENTER>
+static void launch_residual_norm_as(const ResidualNormArgs& a, hipStream_t st) {
+  if (a.top > 0) hipLaunchKernelGGL((residual_norm_kernel<POST, CENTER, true>), dim3(a.T), dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((residual_norm_kernel<POST, CENTER, false>), dim3(a.T), dim3(256), 0, st, a);
+}
+void launch_residual_norm(const ResidualNormArgs& a, hipStream_t st) {
+  if (a.T <= 0 || a.W <= 0) return;
+  if (a.post_w != nullptr) {
+    if (a.center) launch_residual_norm_as<true, true>(a, st);
+    else launch_residual_norm_as<true, false>(a, st);
+  } else {
+    if (a.center) launch_residual_norm_as<false, true>(a, st);
+    else launch_residual_norm_as<false, false>(a, st);
+  }
 }
 
 void launch_pair_rows(const float* a, const float* b, void* out, int out_f32, int T, int W, hipStream_t st) {
@@ -476,16 +569,16 @@ void launch_post_norm_add(const PostNormArgs& a, hipStream_t st) {
 }
 
 void launch_norm_rows(const void* x, int64_t ldx_, int x_f32, const int32_t* rows, const float* w, int w_scalar,
-                      float eps, void* y, int64_t ldy, int y_f32, int M, int n, hipStream_t st) {
+                      float eps, int center, void* y, int64_t ldy, int y_f32, int M, int n, hipStream_t st) {
   if (M <= 0) return;
-  hipLaunchKernelGGL(norm_rows_kernel, dim3(M), dim3(256), 0, st, x, ldx_, x_f32, rows, w, w_scalar, eps, y, ldy,
+  hipLaunchKernelGGL(norm_rows_kernel, dim3(M), dim3(256), 0, st, x, ldx_, x_f32, rows, w, w_scalar, eps, center, y, ldy,
                      y_f32, n);
 }
 
-void launch_embed_rows(const int32_t* ids, const int32_t* prev, const void* table, int t_f32, float* x, int T, int W,
-                       int vocab, hipStream_t st) {
+void launch_embed_rows(const int32_t* ids, const int32_t* prev, const void* table, int t_f32, float scale, float* x, int T,
+                       int W, int vocab, hipStream_t st) {
   if (T <= 0) return;
-  hipLaunchKernelGGL(embed_rows_kernel, dim3(T), dim3(256), 0, st, ids, prev, table, t_f32, x, W, vocab);
+  hipLaunchKernelGGL(embed_rows_kernel, dim3(T), dim3(256), 0, st, ids, prev, table, t_f32, scale, x, W, vocab);
 }
 
 void launch_gated_residual(float* x, const void* y1, const void* g1, int64_t ldg1, const float* b1, const void* y2,
@@ -494,15 +587,15 @@ void launch_gated_residual(float* x, const void* y1, const void* g1, int64_t ldg
   hipLaunchKernelGGL(gated_residual_kernel, dim3(T), dim3(256), 0, st, x, y1, g1, ldg1, b1, y2, g2, ldg2, b2, f32, W);
 }
 
-void launch_moe_route(const float* z, const float* corr, int T, int E, int top, float norm_eps, int softmax, float scale,
+void launch_moe_route(const float* z, const float* corr, int T, int E, int top, float norm_eps, int score, float scale,
                       int32_t* idx, float* wts, hipStream_t st) {
   if (T <= 0) return;
   if (E <= 64 * RPL && top <= 64) {
-    hipLaunchKernelGGL(moe_route_wave_kernel, dim3((T + 3) / 4), dim3(256), 0, st, z, corr, T, E, top, norm_eps, softmax,
+    hipLaunchKernelGGL(moe_route_wave_kernel, dim3((T + 3) / 4), dim3(256), 0, st, z, corr, T, E, top, norm_eps, score,
                        scale, idx, wts);
     return;
   }
-  hipLaunchKernelGGL(moe_route_kernel, dim3((T + 63) / 64), dim3(64), 0, st, z, corr, T, E, top, norm_eps, softmax, scale,
+  hipLaunchKernelGGL(moe_route_kernel, dim3((T + 63) / 64), dim3(64), 0, st, z, corr, T, E, top, norm_eps, score, scale,
                      idx, wts);
 }
 

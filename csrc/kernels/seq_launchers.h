@@ -24,19 +24,20 @@ struct AnyGemmArgs {
   const int32_t* group_off = nullptr;   // [groups + 1] row ranges (device): rows of group g use W + g * w_bs
   int groups = 0;
   int act = 0;                          // 0 none; 1 silu(g) * u; 2 clamped: g' = min(g, L), u' = clamp(u, -L, L),
-  float limit = 0.f;                    //   g' * sigmoid(alpha g') * (u' + 1); 3 tanh (single matrix);
-                                        //   4 gelu_tanh(g) * u
+  float limit = 0.f;                    //   g' * sigmoid(alpha g') * (u' + 1); 4 gelu_tanh(g) * u; of a single matrix:
+                                        //   3 tanh, 5 gelu (erf form), 6 max(g, 0)^2
   float alpha = 1.702f;
   int in_f32 = 0, out_f32 = 0, gate_f32 = 0;
 };
 void launch_gemm_any(const AnyGemmArgs& g, hipStream_t st);
 
-// y[m][:] = x[row(m)][:] * rsqrt(mean(x^2) + eps) * w   (w: one number if w_scalar, else [n])
+// y[m][:] = x[row(m)][:] * rsqrt(mean(x^2) + eps) * w   (w: one number if w_scalar, else [n]); center: a layer norm, the
+// row's mean is taken off first (the variance is the mean of the squared deviations)
 void launch_norm_rows(const void* x, int64_t ldx, int x_f32, const int32_t* rows, const float* w, int w_scalar,
-                      float eps, void* y, int64_t ldy, int y_f32, int M, int n, hipStream_t st);
-// x[t][:] = table[id(t)][:] as fp32; ids < 0 name the previous step's sample prev[-id - 1]
-void launch_embed_rows(const int32_t* ids, const int32_t* prev, const void* table, int t_f32, float* x, int T, int W,
-                       int vocab, hipStream_t st);
+                      float eps, int center, void* y, int64_t ldy, int y_f32, int M, int n, hipStream_t st);
+// x[t][:] = table[id(t)][:] * scale as fp32; ids < 0 name the previous step's sample prev[-id - 1]
+void launch_embed_rows(const int32_t* ids, const int32_t* prev, const void* table, int t_f32, float scale, float* x, int T,
+                       int W, int vocab, hipStream_t st);
 // x += y1 * sigmoid(g1 + b1) [+ y2 * sigmoid(g2 + b2)]; null g: plain add
 void launch_gated_residual(float* x, const void* y1, const void* g1, int64_t ldg1, const float* b1, const void* y2,
                            const void* g2, int64_t ldg2, const float* b2, int f32, int T, int W, hipStream_t st);
@@ -47,9 +48,22 @@ void launch_cast_rows(const float* x, void* y, int T, int n, hipStream_t st);
 // 2 clamped: g' = min(g, limit), g' * sigmoid(alpha g') * (clamp(u, -limit, limit) + 1)
 void launch_glu_rows(const void* gu, int64_t ldg, void* out, int64_t ldo, int T, int n, int act, float limit, float alpha,
                      hipStream_t st);
-// x[t] += mult * y[t] in fp32 (x [T][W]); with w [W]: h[t] = x[t] * rsqrt(mean(x[t]^2) + eps) * w from the new row
-void launch_residual_norm(float* x, const void* y, int y_f32, float mult, const float* w, float eps, void* h, int h_f32,
-                          int T, int W, hipStream_t st);
+// out[t][j] = act(x[t][j]) (bf16 rows, n % 8 == 0, 16-B aligned, out may be x); act 3 tanh, 5 gelu (erf form), 6 max(x, 0)^2
+void launch_act_rows(const void* x, int64_t ldx, void* out, int64_t ldo, int T, int n, int act, hipStream_t st);
+// x[t] += mult * u[t] in fp32 (x [T][W]); with w [W]: h[t] = norm(x[t]) * w from the new row. u[t] = y[t], or with top > 0
+// the weighted sum of a token's expert rows sum_c wts[t][c] * y[pos[t][c]]; with post_w [W]: u[t] = norm(.) * post_w.
+// norm: divided by sqrt(mean(.^2) + eps), with `center` after the row's mean is taken off (layer norm)
+struct ResidualNormArgs {
+  float* x = nullptr;
+  const void* y = nullptr; int y_f32 = 0;
+  const int32_t* pos = nullptr; const float* wts = nullptr; int top = 0;
+  float mult = 1.f, eps = 0.f;
+  const float* post_w = nullptr; const float* w = nullptr;
+  int center = 0;
+  void* h = nullptr; int h_f32 = 0;
+  int T = 0, W = 0;
+};
+void launch_residual_norm(const ResidualNormArgs& a, hipStream_t st);
 // out[t] = [a[t], b[t]] (fp32 rows of W side by side) in out's dtype
 void launch_pair_rows(const float* a, const float* b, void* out, int out_f32, int T, int W, hipStream_t st);
 // out[k][t] = h[t] + (h'[t] - h[t]) * mu[k] for k < n blend vectors mu [n][W] (plane: stride between out's k planes),
@@ -126,6 +140,7 @@ struct WindowArgs {
   float cap_in = 0.f, cap_out = 0.f;    // (set by launch_window_attn: 2 / c and c log2 e)
   int page = 0, npool = 0;              // tokens per page; pooled rows per page (0: no pooled caches)
   int rot_dims = 0, window = 0, pool = 0;
+  int chunk = 0;                        // c > 0: position i sees only j with floor(j / c) = floor(i / c) (not with pooled blocks)
   int f32 = 0, T = 0, S = 0, max_blocks = 0;
   int prefill_kernel = 0;               // MFMA path, prompt portions: 0 LDS-staged tiles (64 rows), 1 split tiles (16 rows)
   const float* inv_freq = nullptr;      // [rot_dims / 2]
@@ -148,17 +163,20 @@ struct WindowArgs {
 size_t window_attn_lds_bytes(const WindowArgs& a, int heads_per_block);
 // how many workgroups share a decoded token's key tiles (1: no split; only the bf16 MFMA kernel splits), and the
 // fp32 scratch elements window_attn then needs
-int window_attn_parts(int T, int S, int H, int G, int D, int V, int f32, int page);
+// (span: the most keys a position sees, 0 = not bounded)
+int window_attn_parts(int T, int S, int H, int G, int D, int V, int f32, int page, int span);
 int window_attn_nct(int D, int V);   // 16-column value tiles of the MFMA kernel instantiation for these head sizes
 size_t window_attn_part_floats(int T, int S, int H, int G, int D, int V, int parts);
 bool window_attn_fits(const WindowArgs& a);   // sizes the kernels' LDS and register budgets take
 // q / k norm (qw, kw null: none; norm_all: one norm over the whole projection) + rotation + paged stores; q_out [T][H * D];
 // the query of head h at position p is multiplied by q_head_scale[h] (null: 1) * (1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1));
 // vt: optional second, transposed bf16 copy of the values [pages][GV][V][page]; rot_half: entry i is paired with
-// entry i + rot_dims / 2 instead of 2i with 2i + 1
+// entry i + rot_dims / 2 instead of 2i with 2i + 1; v_other (rows of GV * V, stride ldo): the values become
+// (1 - lam) v + lam v_other in fp32 before anything else happens to them
 void launch_window_write(const WindowArgs& a, const void* q, int64_t ldq, const void* k, int64_t ldk, const void* v,
                          int64_t ldv, const float* qw, const float* kw, float eps, int norm_all, void* q_out, void* vt,
-                         const float* q_head_scale, float q_temp_coef, int q_temp_every, int rot_half, hipStream_t st);
+                         const float* q_head_scale, float q_temp_coef, int q_temp_every, int rot_half, const void* v_other,
+                         int64_t ldo, float lam, hipStream_t st);
 // pooled rows of the blocks this step's tokens complete
 void launch_window_pool(const WindowArgs& a, hipStream_t st);
 // out[t][h][:V] = softmax over (pooled blocks before the window, window tokens [, sink]) of scale q . key, times values
@@ -198,9 +216,10 @@ size_t linear_attn_scratch_floats(int T, int S, int H, int D, int V);
 // T rows; scratch: linear_attn_scratch_floats() floats, 16-B aligned
 void launch_linear_attn(const LinearAttnArgs& a, int T, float* scratch, hipStream_t st);
 
-// idx, wts [T][top]: the `top` largest of s + corr with s = sigmoid(z) or, with `softmax`, softmax(z) over all E;
-// wts = s of the chosen / (their sum + norm_eps) * scale
-void launch_moe_route(const float* z, const float* corr, int T, int E, int top, float norm_eps, int softmax, float scale,
+// idx, wts [T][top]: the `top` largest of s + corr with s by `score`: 0 sigmoid(z), 1 softmax(z) over all E;
+// wts = s of the chosen / (their sum + norm_eps) * scale. score 2: the `top` largest of z + corr, wts = softmax of z over
+// the chosen alone, times scale
+void launch_moe_route(const float* z, const float* corr, int T, int E, int top, float norm_eps, int score, float scale,
                       int32_t* idx, float* wts, hipStream_t st);
 // counting sort of the T * top (token, choice) pairs by expert: rows[p] = token, pos[t * top + c] = p,
 // off[E + 1] = group boundaries

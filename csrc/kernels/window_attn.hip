@@ -37,8 +37,14 @@
 // Softcap c > 0 (not with a distance term): the scaled score s becomes c tanh(s / c) (CAP instantiations of the MFMA
 //               kernels). The value caches may have fewer heads (GV) than the key cache: key head g reads value head
 //               g / (G / GV), which is how two score maps of one head share their values.
+// Chunks (c > 0, not with pooled blocks): position i sees only the keys of its own chunk of c positions, counted from
+//               position 0 (first_key()); with a window too, the nearer of the two bounds holds. The key tiles a workgroup
+//               walks start at the chunk of its first row.
+// Value mixing: window_write can blend a token's values with another row of values of the same token (fp32).
 // Every row of every kernel depends only on its own sequence's cache rows, in an order fixed by the
 // position, so results do not depend on how a prompt is cut or what else is in the batch.
+#include <algorithm>
+
 #include "common.h"
 #include "seq_launchers.h"
 
@@ -62,13 +68,20 @@ __device__ __forceinline__ int seq_of_token(const int32_t* query_start, int S, i
   return lo;
 }
 
+// the first position the query at position p sees (may be negative without chunks: no bound); never decreases with p
+__device__ __forceinline__ int first_key(const WindowArgs& a, int p) {
+  const int lo = p - a.window + 1;
+  return a.chunk > 0 ? max(lo, p - p % a.chunk) : lo;
+}
+
 __global__ __launch_bounds__(256) void window_write_kernel(WindowArgs a, const void* __restrict__ q, int64_t ldq,
                                                             const void* __restrict__ k, int64_t ldk,
                                                             const void* __restrict__ v, int64_t ldv,
                                                             const float* __restrict__ qw, const float* __restrict__ kw,
                                                             float eps, int norm_all, void* __restrict__ q_out,
                                                             bf16_t* __restrict__ vt, const float* __restrict__ q_head_scale,
-                                                            float q_temp_coef, int q_temp_every, int rot_half) {
+                                                            float q_temp_coef, int q_temp_every, int rot_half,
+                                                            const void* __restrict__ v_other, int64_t ldo, float lam) {
   extern __shared__ float lds[];
   const int H = a.H, G = a.G, D = a.D, V = a.V, GV = a.GV;
   float* xs = lds;                    // [(H + G) * D] q heads then k heads
@@ -128,16 +141,20 @@ __global__ __launch_bounds__(256) void window_write_kernel(WindowArgs a, const v
     else stx(a.kc, ((pg * G + (h - H)) * page + off) * D + i, a.f32, o);
   }
   const int vrot = a.v_freq != nullptr ? 2 * (V / 2) : 0;
+  auto val = [&](int e) {  // entry e of the token's values, blended with the other row's
+    const float x = ldx(v, (int64_t)t * ldv + e, a.f32);
+    return v_other != nullptr ? fmaf(lam, ldx(v_other, (int64_t)t * ldo + e, a.f32), (1.f - lam) * x) : x;
+  };
   for (int e = tid; e < GV * V; e += 256) {
     const int g = e / V, i = e % V;
     float o;
     if (i < vrot) {
-      const float x0 = ldx(v, (int64_t)t * ldv + g * V + (i & ~1), a.f32), x1 = ldx(v, (int64_t)t * ldv + g * V + (i | 1), a.f32);
+      const float x0 = val(g * V + (i & ~1)), x1 = val(g * V + (i | 1));
       const float ang = pos * a.v_freq[i >> 1];
       const float cs = cosf(ang), sn = sinf(ang);
       o = (i & 1) ? (x1 * cs + x0 * sn) : (x0 * cs - x1 * sn);
     } else {
-      o = ldx(v, (int64_t)t * ldv + e, a.f32);
+      o = val(e);
     }
     stx(a.vc, ((pg * GV + g) * page + off) * V + i, a.f32, o);
     if (vt != nullptr) vt[((pg * GV + g) * V + i) * page + off] = f2bf(o);  // [page][GV][column][key in page]
@@ -226,7 +243,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowArgs a, const vo
   const int nh = min(HC, rep - r0);
   const int h0 = g * rep + r0;
   const int tid = threadIdx.x;
-  const int lo = max(0, pos - a.window + 1);
+  const int lo = max(0, first_key(a, pos));
   const int nb = a.pool > 0 ? max(0, pos - a.window + 1) / a.pool : 0;  // pooled blocks wholly before the window
   const int nkeys = nb + (pos - lo + 1);
   for (int e = tid; e < nh * D; e += 256) qs[(e / D) * DP + e % D] = ldx(q, ((int64_t)t * a.H + h0) * D + e, a.f32);
@@ -489,7 +506,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(WindowArgs a,
     const bool ok = r < nrows;
     const int p = pos0 + (ok ? r / rep : 0);
     hi[i] = ok ? p : -1;
-    lo[i] = p - a.window + 1;
+    lo[i] = first_key(a, p);
     nbv[i] = (ok && P > 0) ? max(0, lo[i]) / P : 0;
     if (BIAS) {
       bias_row(a, g, rep, r, ok, bw[i], bx[i], bo[i]);
@@ -501,7 +518,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(WindowArgs a,
   }
   const int last = min(row0 + 15, nrows - 1);
   const int pmin = pos0 + row0 / rep, pmax = pos0 + last / rep;  // wave-uniform
-  const int klo = max(0, pmin - a.window + 1);
+  const int klo = max(0, first_key(a, pmin));
   const int nbmax = P > 0 ? max(0, pmax - a.window + 1) / P : 0;
   const int ntp = (nbmax + 31) >> 5, jt0 = klo >> 5;
   const int ntiles = ntp + (pmax >> 5) - jt0 + 1;
@@ -809,7 +826,7 @@ __global__ __launch_bounds__(256) void window_attn_tiled_kernel(WindowArgs a, co
     const bool ok = r < nrows;
     const int p = pos0 + (ok ? r / rep : 0);
     hi[i] = ok ? p : -1;
-    lo[i] = p - a.window + 1;
+    lo[i] = first_key(a, p);
     nbv[i] = (ok && P > 0) ? max(0, lo[i]) / P : 0;
     if (BIAS) {
       bias_row(a, g, rep, r, ok, bw[i], bx[i], bo[i]);
@@ -822,11 +839,11 @@ __global__ __launch_bounds__(256) void window_attn_tiled_kernel(WindowArgs a, co
   // workgroup-uniform key ranges
   const int lastb = min(rowb + 63, nrows - 1);
   const int pminb = pos0 + rowb / rep, pmaxb = pos0 + lastb / rep;
-  const int jt0 = max(0, pminb - a.window + 1) >> 5, jt1 = pmaxb >> 5;
+  const int jt0 = max(0, first_key(a, pminb)) >> 5, jt1 = pmaxb >> 5;
   // wave-uniform: what this wave's rows can see at all
   const int lastw = min(row0 + 15, nrows - 1);
   const int pminw = pos0 + row0 / rep, pmaxw = pos0 + lastw / rep;
-  const int klow = max(0, pminw - a.window + 1);
+  const int klow = max(0, first_key(a, pminw));
   const int nbmax = (active && P > 0) ? max(0, pmaxw - a.window + 1) / P : 0;
   f32x4 O[NCT];
 #pragma unroll
@@ -1041,11 +1058,13 @@ int heads_per_block(const WindowArgs& a) {
 
 // Decoded tokens on the MFMA kernel: how many workgroups share the key tiles of a 16-row tile (1: no split) so that
 // the launch has about two workgroups of eight waves per CU, and the scratch floats their partial results take.
-int window_attn_parts(int T, int S, int H, int G, int D, int V, int f32, int page) {
+// span > 0: no position sees more keys than that (no more workgroups than its tiles of 32 keys fill, at one per wave).
+int window_attn_parts(int T, int S, int H, int G, int D, int V, int f32, int page, int span) {
   const int rep = H / G;
   if (f32 || page != 16 || D % 8 != 0 || D < 8 || D > 256 || V > 256 || (int64_t)T * rep > 16 * (int64_t)S) return 1;
   const int wg = ((T * rep + 15) / 16 + S) * G;
-  const int parts = 512 / (wg > 0 ? wg : 1);
+  int parts = 512 / (wg > 0 ? wg : 1);
+  if (span > 0) parts = std::min(parts, (span / 32 + 1 + 7) / 8);
   return parts < 2 ? 1 : (parts > 8 ? 8 : parts);
 }
 int window_attn_nct(int D, int V) { return (D <= 64 && V <= 64) ? 4 : ((D <= 128 && V <= 128) ? 8 : 16); }
@@ -1067,11 +1086,12 @@ bool window_attn_fits(const WindowArgs& a) {
 
 void launch_window_write(const WindowArgs& a, const void* q, int64_t ldq, const void* k, int64_t ldk, const void* v,
                          int64_t ldv, const float* qw, const float* kw, float eps, int norm_all, void* q_out, void* vt,
-                         const float* q_head_scale, float q_temp_coef, int q_temp_every, int rot_half, hipStream_t st) {
+                         const float* q_head_scale, float q_temp_coef, int q_temp_every, int rot_half, const void* v_other,
+                         int64_t ldo, float lam, hipStream_t st) {
   if (a.T <= 0) return;
   const size_t lds = (size_t)((a.H + a.G) * a.D + a.H + a.G) * sizeof(float);
   hipLaunchKernelGGL(window_write_kernel, dim3(a.T), dim3(256), lds, st, a, q, ldq, k, ldk, v, ldv, qw, kw, eps, norm_all,
-                     q_out, reinterpret_cast<bf16_t*>(vt), q_head_scale, q_temp_coef, q_temp_every, rot_half);
+                     q_out, reinterpret_cast<bf16_t*>(vt), q_head_scale, q_temp_coef, q_temp_every, rot_half, v_other, ldo, lam);
 }
 
 void launch_window_pool(const WindowArgs& a, hipStream_t st) {

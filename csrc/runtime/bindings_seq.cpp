@@ -68,7 +68,7 @@ void gemm_any(const Tensor& a, const Tensor& w, Tensor& out, const OptT& w2, con
     g.w2 = w2->data_ptr();
     TORCH_CHECK(act == 1 || act == 2 || act == 4, "gemm_any: a weight pair needs act 1, 2 or 4");
   } else {
-    TORCH_CHECK(act == 0 || act == 3, "gemm_any: act 1 / 2 / 4 need a weight pair");
+    TORCH_CHECK(act == 0 || act == 3 || act == 5 || act == 6, "gemm_any: act 1 / 2 / 4 need a weight pair");
   }
   g.bias = f32p(bias, "bias", g.N);
   TORCH_CHECK(!(g.bias && B > 1), "gemm_any: bias only without batch");
@@ -94,7 +94,7 @@ void gemm_any(const Tensor& a, const Tensor& w, Tensor& out, const OptT& w2, con
   vgate::launch_gemm_any(g, cur_stream());
 }
 
-void norm_rows(const Tensor& x, const Tensor& w, double eps, Tensor& y, const OptT& rows, bool scalar) {
+void norm_rows(const Tensor& x, const Tensor& w, double eps, Tensor& y, const OptT& rows, bool scalar, bool center) {
   const int xf = act_f32(x, "x"), yf = act_f32(y, "y");
   TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && x.size(1) == y.size(1), "norm_rows: [M, n] rows");
   const int64_t n = x.size(1), M = y.size(0);
@@ -103,11 +103,11 @@ void norm_rows(const Tensor& x, const Tensor& w, double eps, Tensor& y, const Op
   if (has(rows)) rp = i32p(*rows, "rows", M);
   else TORCH_CHECK(x.size(0) >= M, "norm_rows: x rows");
   c10::DeviceGuard guard(x.device());
-  vgate::launch_norm_rows(x.data_ptr(), x.stride(0), xf, rp, wp, scalar ? 1 : 0, (float)eps, y.data_ptr(), y.stride(0),
-                          yf, (int)M, (int)n, cur_stream());
+  vgate::launch_norm_rows(x.data_ptr(), x.stride(0), xf, rp, wp, scalar ? 1 : 0, (float)eps, center ? 1 : 0, y.data_ptr(),
+                          y.stride(0), yf, (int)M, (int)n, cur_stream());
 }
 
-void embed_rows(const Tensor& ids, const Tensor& table, Tensor& x, const OptT& prev) {
+void embed_rows(const Tensor& ids, const Tensor& table, Tensor& x, const OptT& prev, double scale) {
   const int tf = act_f32(table, "table");
   TORCH_CHECK(table.dim() == 2 && table.is_contiguous(), "embed_rows: table [vocab, W]");
   TORCH_CHECK(x.is_cuda() && x.scalar_type() == torch::kFloat32 && x.is_contiguous() && x.dim() == 2 &&
@@ -116,8 +116,8 @@ void embed_rows(const Tensor& ids, const Tensor& table, Tensor& x, const OptT& p
   const int32_t* ip = i32p(ids, "ids", T);
   const int32_t* pp = has(prev) ? i32p(*prev, "prev", 1) : nullptr;
   c10::DeviceGuard guard(x.device());
-  vgate::launch_embed_rows(ip, pp, table.data_ptr(), tf, x.data_ptr<float>(), T, (int)x.size(1), (int)table.size(0),
-                           cur_stream());
+  vgate::launch_embed_rows(ip, pp, table.data_ptr(), tf, (float)scale, x.data_ptr<float>(), T, (int)x.size(1),
+                           (int)table.size(0), cur_stream());
 }
 
 void gated_residual(Tensor& x, const Tensor& y1, const OptT& g1, const OptT& b1, const OptT& y2, const OptT& g2,
@@ -287,23 +287,49 @@ void glu_rows(const Tensor& gu, Tensor& out, int64_t act, double limit, double a
                          (float)limit, (float)alpha, cur_stream());
 }
 
-void residual_norm(Tensor& x, const Tensor& y, double mult, const OptT& w, double eps, const OptT& h_out) {
+void act_rows(const Tensor& x, Tensor& out, int64_t act) {
+  for (const Tensor* t : {&x, const_cast<const Tensor*>(&out)})
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == torch::kBFloat16 && t->dim() == 2 && t->stride(1) == 1 &&
+                t->stride(0) % 8 == 0 && (reinterpret_cast<uintptr_t>(t->data_ptr()) & 15) == 0,
+                "act_rows: bf16 rows of whole 16-B pieces");
+  TORCH_CHECK(out.size(0) <= x.size(0) && out.size(1) == x.size(1) && out.size(1) % 8 == 0, "act_rows: out [<= T, n], n a multiple of 8");
+  TORCH_CHECK(act == 3 || act == 5 || act == 6, "act_rows: act 3 (tanh), 5 (gelu) or 6 (squared relu)");
+  c10::DeviceGuard guard(x.device());
+  vgate::launch_act_rows(x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0), (int)out.size(0), (int)out.size(1), (int)act,
+                         cur_stream());
+}
+
+// pos / wts [T * top]: y then is [T * top, W], a token's expert rows
+void residual_norm(Tensor& x, const Tensor& y, double mult, const OptT& w, double eps, const OptT& h_out, const OptT& post_w,
+                   bool center, const OptT& pos, const OptT& wts) {
   TORCH_CHECK(x.is_cuda() && x.scalar_type() == torch::kFloat32 && x.is_contiguous() && x.dim() == 2, "residual_norm: x fp32 [T, W]");
-  const int yf = act_f32(y, "y");
-  const int64_t T = y.size(0), W = x.size(1);
-  TORCH_CHECK(y.dim() == 2 && y.is_contiguous() && y.size(1) == W && T <= x.size(0), "residual_norm: y [<= T, W]");
-  const float* wp = f32p(w, "w", W);
-  void* hp = nullptr;
-  int hf = 0;
+  vgate::ResidualNormArgs a;
+  a.y_f32 = act_f32(y, "y");
+  const int64_t W = x.size(1);
+  int64_t T = y.size(0);
+  TORCH_CHECK(y.dim() == 2 && y.is_contiguous() && y.size(1) == W, "residual_norm: y rows of W");
+  TORCH_CHECK(has(pos) == has(wts), "residual_norm: pos and wts come together");
+  if (has(pos)) {
+    TORCH_CHECK(wts->dim() == 2 && wts->size(0) * wts->size(1) == T && pos->numel() == T, "residual_norm: pos / wts [T, top], y [T * top, W]");
+    T = wts->size(0);
+    a.top = (int)wts->size(1);
+    a.pos = i32p(*pos, "pos", T * a.top);  // values < T * top: a permutation made by moe_sort
+    a.wts = f32p(wts, "wts", T * a.top);
+  }
+  TORCH_CHECK(T <= x.size(0), "residual_norm: x has fewer rows than y");
+  a.x = x.data_ptr<float>(); a.y = y.data_ptr(); a.mult = (float)mult; a.eps = (float)eps;
+  a.w = f32p(w, "w", W);
+  a.post_w = f32p(post_w, "post_w", W);
+  a.center = center ? 1 : 0;
   TORCH_CHECK(has(w) == has(h_out), "residual_norm: the norm weight and its output come together");
   if (has(h_out)) {
-    hf = act_f32(*h_out, "h_out");
+    a.h_f32 = act_f32(*h_out, "h_out");
     TORCH_CHECK(h_out->dim() == 2 && h_out->is_contiguous() && h_out->size(1) == W && h_out->size(0) >= T, "residual_norm: h_out [T, W]");
-    hp = h_out->data_ptr();
+    a.h = h_out->data_ptr();
   }
+  a.T = (int)T; a.W = (int)W;
   c10::DeviceGuard guard(x.device());
-  vgate::launch_residual_norm(x.data_ptr<float>(), y.data_ptr(), yf, (float)mult, wp, (float)eps, hp, hf, (int)T, (int)W,
-                              cur_stream());
+  vgate::launch_residual_norm(a, cur_stream());
 }
 
 void pair_rows(const Tensor& a, const Tensor& b, Tensor& out) {
@@ -437,7 +463,8 @@ void* window_vt(const OptT& vt, const Tensor& vc) {
 void window_write(const Tensor& q, const Tensor& k, const Tensor& v, const OptT& qw, const OptT& kw, double eps,
                   bool norm_all, const Tensor& positions, const Tensor& slots, const Tensor& inv_freq, int64_t rot_dims,
                   const OptT& v_freq, Tensor& kc, Tensor& vc, Tensor& q_out, int64_t H, int64_t G, const OptT& vt,
-                  const OptT& q_head_scale, double q_temp_coef, int64_t q_temp_every, bool rot_half) {
+                  const OptT& q_head_scale, double q_temp_coef, int64_t q_temp_every, bool rot_half, const OptT& v_other,
+                  double lam) {
   auto a = window_common(kc, vc, c10::nullopt, c10::nullopt, H, 0);
   TORCH_CHECK(q_temp_every >= 1, "window_write: q_temp_every >= 1");
   TORCH_CHECK(G == a.G, "window_write: kv heads");
@@ -460,10 +487,17 @@ void window_write(const Tensor& q, const Tensor& k, const Tensor& v, const OptT&
   const float* qwp = f32p(qw, "qw", norm_all ? H * a.D : a.D);
   const float* kwp = f32p(kw, "kw", norm_all ? G * a.D : a.D);
   void* vtp = window_vt(vt, vc);
+  const void* vo = nullptr;
+  int64_t ldo = 0;
+  if (has(v_other)) {
+    TORCH_CHECK(act_f32(*v_other, "v_other") == a.f32 && v_other->dim() == 2 && v_other->size(0) >= T &&
+                v_other->size(1) == v.size(1), "window_write: v_other rows like v's");
+    vo = v_other->data_ptr(); ldo = v_other->stride(0);
+  }
   c10::DeviceGuard guard(q.device());
   vgate::launch_window_write(a, q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), qwp, kwp,
                              (float)eps, norm_all ? 1 : 0, q_out.data_ptr(), vtp, f32p(q_head_scale, "q_head_scale", H),
-                             (float)q_temp_coef, (int)q_temp_every, rot_half ? 1 : 0, cur_stream());
+                             (float)q_temp_coef, (int)q_temp_every, rot_half ? 1 : 0, vo, ldo, (float)lam, cur_stream());
 }
 
 void window_seq_meta(vgate::WindowArgs& a, const Tensor& block_tables, const Tensor& query_start) {
@@ -488,8 +522,10 @@ void window_attn(const Tensor& q, const Tensor& kc, const Tensor& vc, const OptT
                  const Tensor& block_tables, const Tensor& context_lens, const Tensor& query_start, Tensor& out,
                  double scale, int64_t H, int64_t window, int64_t pool, const OptT& sink, const OptT& v_freq, const OptT& vt,
                  int64_t prefill_kernel, int64_t bias_kind, const OptT& bias_a, const OptT& bias_b, const OptT& gate,
-                 int64_t parts, const OptT& part_scratch, double softcap) {
+                 int64_t parts, const OptT& part_scratch, double softcap, int64_t chunk) {
   auto a = window_common(kc, vc, kp, vp, H, pool);
+  TORCH_CHECK(chunk >= 0 && chunk <= (1 << 30) && (chunk == 0 || pool == 0), "window_attn: chunk 0 (none) .. 2^30, not with pooled blocks");
+  a.chunk = (int)chunk;
   TORCH_CHECK(softcap >= 0.0 && (softcap == 0.0 || bias_kind == 0), "window_attn: softcap >= 0, not with a distance term");
   a.softcap = (float)softcap;
   window_seq_meta(a, block_tables, query_start);
@@ -526,7 +562,7 @@ void window_attn(const Tensor& q, const Tensor& kc, const Tensor& vc, const OptT
   a.v_freq = f32p(v_freq, "v_freq", a.V / 2);
   const void* vtp = window_vt(vt, vc);
   if (parts > 1) {  // only what window_attn_parts() allows for this launch, with its scratch
-    TORCH_CHECK(vtp != nullptr && parts == vgate::window_attn_parts((int)T, a.S, a.H, a.G, a.D, a.V, a.f32, a.page),
+    TORCH_CHECK(vtp != nullptr && parts == vgate::window_attn_parts((int)T, a.S, a.H, a.G, a.D, a.V, a.f32, a.page, a.chunk),
                 "window_attn: parts must be window_attn_split()'s for this step");
     const size_t need = vgate::window_attn_part_floats((int)T, a.S, a.H, a.G, a.D, a.V, (int)parts);
     TORCH_CHECK(has(part_scratch) && part_scratch->is_cuda() && part_scratch->scalar_type() == torch::kFloat32 &&
@@ -601,8 +637,9 @@ void linear_attn(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor
   vgate::launch_linear_attn(p, (int)T, scratch.data_ptr<float>(), cur_stream());
 }
 
-void moe_route(const Tensor& z, const OptT& corr, int64_t top, double norm_eps, Tensor& idx, Tensor& wts, bool softmax,
+void moe_route(const Tensor& z, const OptT& corr, int64_t top, double norm_eps, Tensor& idx, Tensor& wts, int64_t score,
                double scale) {
+  TORCH_CHECK(score >= 0 && score <= 2, "moe_route: score 0 (sigmoid), 1 (softmax) or 2 (softmax over the chosen)");
   TORCH_CHECK(z.is_cuda() && z.scalar_type() == torch::kFloat32 && z.is_contiguous() && z.dim() == 2, "moe_route: z fp32 [T, E]");
   const int64_t T = z.size(0), E = z.size(1);
   TORCH_CHECK(top >= 1 && top <= E, "moe_route: top");
@@ -610,7 +647,7 @@ void moe_route(const Tensor& z, const OptT& corr, int64_t top, double norm_eps, 
   TORCH_CHECK(wts.is_cuda() && wts.scalar_type() == torch::kFloat32 && wts.is_contiguous() && wts.numel() == T * top, "moe_route: wts");
   c10::DeviceGuard guard(z.device());
   vgate::launch_moe_route(z.data_ptr<float>(), f32p(corr, "corr", E), (int)T, (int)E, (int)top, (float)norm_eps,
-                          softmax ? 1 : 0, (float)scale, idx.data_ptr<int32_t>(), wts.data_ptr<float>(), cur_stream());
+                          (int)score, (float)scale, idx.data_ptr<int32_t>(), wts.data_ptr<float>(), cur_stream());
 }
 
 void moe_sort(const Tensor& idx, int64_t E, Tensor& rows, Tensor& pos, Tensor& off) {
@@ -703,10 +740,11 @@ void bind_seq(pybind11::module& m) {
         py::arg("a"), py::arg("w"), py::arg("out"), py::arg("w2") = py::none(), py::arg("bias") = py::none(),
         py::arg("gate") = py::none(), py::arg("a_rows") = py::none(), py::arg("group_off") = py::none(),
         py::arg("act") = 0, py::arg("limit") = 0.0, py::arg("alpha") = 1.702);
-  m.def("norm_rows", &norm_rows, "RMS norm of rows, scalar or vector weight, fp32 statistics", py::arg("x"), py::arg("w"),
-        py::arg("eps"), py::arg("y"), py::arg("rows") = py::none(), py::arg("scalar") = false);
+  m.def("norm_rows", &norm_rows, "RMS or (center) layer norm of rows, scalar or vector weight, fp32 statistics", py::arg("x"),
+        py::arg("w"), py::arg("eps"), py::arg("y"), py::arg("rows") = py::none(), py::arg("scalar") = false,
+        py::arg("center") = false);
   m.def("embed_rows", &embed_rows, "embedding gather into the fp32 residual stream", py::arg("ids"), py::arg("table"),
-        py::arg("x"), py::arg("prev") = py::none());
+        py::arg("x"), py::arg("prev") = py::none(), py::arg("scale") = 1.0);
   m.def("gated_residual", &gated_residual, "x += y1 * sigmoid(g1 + b1) + y2 * sigmoid(g2 + b2)", py::arg("x"),
         py::arg("y1"), py::arg("g1") = py::none(), py::arg("b1") = py::none(), py::arg("y2") = py::none(),
         py::arg("g2") = py::none(), py::arg("b2") = py::none());
@@ -727,9 +765,13 @@ void bind_seq(pybind11::module& m) {
   m.def("cast_rows", &cast_rows, "fp32 rows rounded to bf16");
   m.def("glu_rows", &glu_rows, "out = act(gate) * up over a stacked [gate; up] projection", py::arg("gu"), py::arg("out"),
         py::arg("act"), py::arg("limit") = 0.0, py::arg("alpha") = 1.702);
-  m.def("residual_norm", &residual_norm, "x += mult * y in fp32, and the RMS norm of the new rows for the next sublayer",
+  m.def("act_rows", &act_rows, "out = act(x) over bf16 rows", py::arg("x"), py::arg("out"), py::arg("act"));
+  m.def("residual_norm", &residual_norm,
+        "x += mult * (y, or a token's weighted expert rows; optionally normed first) in fp32, and the norm of the new rows "
+        "for the next sublayer",
         py::arg("x"), py::arg("y"), py::arg("mult"), py::arg("w") = py::none(), py::arg("eps") = 0.0,
-        py::arg("h_out") = py::none());
+        py::arg("h_out") = py::none(), py::arg("post_w") = py::none(), py::arg("center") = false, py::arg("pos") = py::none(),
+        py::arg("wts") = py::none());
   m.def("pair_rows", &pair_rows, "two fp32 row sets side by side in the activation dtype");
   m.def("shift_mix", &shift_mix, "blends of every token's row with the row of the token before it; keeps the last row");
   m.def("map_pair_combine", &map_pair_combine, "two attention maps per head: a1 - lam a2, head RMS norm, scale, gate");
@@ -741,16 +783,18 @@ void bind_seq(pybind11::module& m) {
         py::arg("k"), py::arg("v"), py::arg("qw"), py::arg("kw"), py::arg("eps"), py::arg("norm_all"), py::arg("positions"),
         py::arg("slots"), py::arg("inv_freq"), py::arg("rot_dims"), py::arg("v_freq"), py::arg("kc"), py::arg("vc"),
         py::arg("q_out"), py::arg("H"), py::arg("G"), py::arg("vt") = py::none(), py::arg("q_head_scale") = py::none(),
-        py::arg("q_temp_coef") = 0.0, py::arg("q_temp_every") = 1, py::arg("rot_half") = false);
+        py::arg("q_temp_coef") = 0.0, py::arg("q_temp_every") = 1, py::arg("rot_half") = false,
+        py::arg("v_other") = py::none(), py::arg("lam") = 0.0);
   m.def("window_pool", &window_pool, "mean key / value rows of the blocks a step completes");
   m.def("window_attn", &window_attn, "sliding-window attention with pooled blocks and an optional sink", py::arg("q"),
         py::arg("kc"), py::arg("vc"), py::arg("kp"), py::arg("vp"), py::arg("block_tables"), py::arg("context_lens"),
         py::arg("query_start"), py::arg("out"), py::arg("scale"), py::arg("H"), py::arg("window"), py::arg("pool"),
         py::arg("sink"), py::arg("v_freq"), py::arg("vt") = py::none(), py::arg("prefill_kernel") = 0,
         py::arg("bias_kind") = 0, py::arg("bias_a") = py::none(), py::arg("bias_b") = py::none(), py::arg("gate") = py::none(),
-        py::arg("parts") = 1, py::arg("part_scratch") = py::none(), py::arg("softcap") = 0.0);
-  m.def("window_attn_split", [](int64_t T, int64_t S, int64_t H, int64_t G, int64_t D, int64_t V, bool f32, int64_t page) {
-    const int parts = vgate::window_attn_parts((int)T, (int)S, (int)H, (int)G, (int)D, (int)V, f32 ? 1 : 0, (int)page);
+        py::arg("parts") = 1, py::arg("part_scratch") = py::none(), py::arg("softcap") = 0.0, py::arg("chunk") = 0);
+  m.def("window_attn_split", [](int64_t T, int64_t S, int64_t H, int64_t G, int64_t D, int64_t V, bool f32, int64_t page,
+                                int64_t chunk) {
+    const int parts = vgate::window_attn_parts((int)T, (int)S, (int)H, (int)G, (int)D, (int)V, f32 ? 1 : 0, (int)page, (int)chunk);
     return std::make_pair((int64_t)parts, (int64_t)vgate::window_attn_part_floats((int)T, (int)S, (int)H, (int)G, (int)D, (int)V, parts));
   }, "workgroups that share a decoded token's key tiles in window_attn, and the fp32 scratch elements they need");
   m.def("linear_attn_scratch", [](int64_t T, int64_t S, int64_t H, int64_t D, int64_t V) {
@@ -765,7 +809,7 @@ void bind_seq(pybind11::module& m) {
         py::arg("decay_exp") = false, py::arg("bonus") = py::none(), py::arg("norm_full") = false);
   m.def("moe_route", &moe_route, "sigmoid or softmax router: corrected top-k choice, normalised uncorrected weights, scaled",
         py::arg("z"), py::arg("corr"), py::arg("top"), py::arg("norm_eps"), py::arg("idx"), py::arg("wts"),
-        py::arg("softmax") = false, py::arg("scale") = 1.0);
+        py::arg("score") = 0, py::arg("scale") = 1.0);
   m.def("tanh_norm_rows", &tanh_norm_rows, "tanh(alpha x) * w + b over (gathered) rows");
   m.def("hyper_mix", &hyper_mix, "write of a sublayer to the stream's copies + the next sublayer's normed read + their sum");
   m.def("moe_sort", &moe_sort, "counting sort of (token, choice) pairs by expert");

@@ -643,7 +643,7 @@ def test_softmax_router(device, E, top):
     T, W = 11, 6
     z = 3.0 * torch.randn(T, E, generator=g)
     idx, wts = torch.zeros(T, top, dtype=torch.int32, device=d), torch.zeros(T, top, device=d)
-    seq.moe_route(z.to(d), None, top, 1e-20, idx, wts, softmax=True, scale=1.75)
+    seq.moe_route(z.to(d), None, top, 1e-20, idx, wts, score=seq.ROUTE_SOFTMAX, scale=1.75)
     s = torch.softmax(z.double(), -1)
     ts, ti = torch.topk(s, top, -1)
     assert torch.equal(idx.cpu().long().sort(-1).values, ti.sort(-1).values)

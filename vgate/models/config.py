@@ -139,7 +139,7 @@ class HybridArch:
     hidden_size: int
     vocab_size: int
     layers: tuple
-    rms_eps: float = 1e-6
+    rms_eps: float = 1e-6     # eps of every norm, also where ``norm`` is "layer"
     max_position: int = 1 << 20
     bos_token_id: int = 1
     eos_token_ids: tuple = (2,)
@@ -150,8 +150,11 @@ class HybridArch:
     # copies of the residual stream a layer reads and writes through learned weights (1: one plain stream);
     # the ``hyper_pre_norm`` arrangement uses them
     streams: int = 1
-    # ``pre_norm`` arrangement: every sublayer's result is multiplied by this before it is added
+    # ``pre_norm`` / ``sandwich_norm`` arrangements: every sublayer's result is multiplied by this before it is added;
+    # the norms are "rms" or "layer" (mean taken off, no bias); embedding rows are multiplied by ``embed_scale``
     residual_mult: float = 1.0
+    norm: str = "rms"
+    embed_scale: float = 1.0
     # (start, stop, times): layers start .. stop - 1 run ``times`` times in a row with the same weights, every
     # pass with caches and states of its own; right before the first layer of each pass the stream is replaced by
     # W_in [x; x0] (tensor ``loop.in`` [width, 2 width], x0 the embedding output)
@@ -366,9 +369,50 @@ def _gefudra_from_config(cfg: dict, name: str) -> HybridArch:
                       logit_scale=float(cfg.get("logit_scale", 1.0)), tie_embeddings=True)
 
 
+def _nigozen_mixer(kind: str, m: dict) -> tuple:
+    """(key of ``vgate.models.mixers.MIXERS``, its spec) of a Nigozen layer type. What the design fixes (the pairs the
+    rotation turns, one added to the softmax denominator, the sigmoid gate) is written out here as options."""
+    if kind != "attention":
+        raise ValueError(f"Nigozen has no layer type {kind!r}")
+    rot, mask = m.get("rot") or {}, m.get("mask") or {}
+    size = mask.get("size")
+    return "window_attention", {"heads": int(m["heads"]), "kv_heads": int(m["kv_heads"]), "dim": int(m["dim"]),
+                                "vdim": int(m["vdim"]), "scale": float(m["scale"]), "window": None,
+                                "chunk": None if size is None else int(size),
+                                "rot": {"dims": int(rot.get("dims", 0)), "base": float(rot.get("base", 10000.0)), "layout": "pairs"},
+                                "sink": "one", "gate": "sigmoid", "value_mix": bool(m.get("v_mix", False))}
+
+
+def _nigozen_mlp(mlp: dict | None) -> dict | None:
+    if not mlp:
+        return None
+    if mlp.get("kind") == "dense":
+        return {"kind": "dense", "ff": int(mlp["ff"]), "gated": False, "act": "gelu"}
+    if mlp.get("kind") == "moe":
+        r = mlp["router"]
+        return {"kind": "moe", "expert": {"ff": int(mlp["expert"]["ff"]), "gated": False, "act": "relu2"},
+                "router": {"experts": int(r["experts"]), "top": int(r["top"]), "score": "top_softmax", "correction": False}}
+    raise ValueError(f"Nigozen feed-forward kind {mlp.get('kind')!r}")
+
+
+def _nigozen_from_config(cfg: dict, name: str) -> HybridArch:
+    """config.json of the Nigozen design: layer norms before and after each sublayer, chunked attention whose values
+    are blended with the first such layer's, dense or routed feed-forwards without gates, scaled embedding rows
+    and the embedding table as the output matrix."""
+    layers = []
+    for L in cfg["layers"]:
+        kind, spec = _nigozen_mixer(L["type"], L["mixer"])
+        layers.append(LayerSpec(kind=kind, mixer=spec, mlp=_nigozen_mlp(L.get("mlp"))))
+    eos = cfg.get("eos_token_id", 2)
+    return HybridArch(name=name, family="nigozen", hidden_size=int(cfg["width"]), vocab_size=int(cfg["vocab"]),
+                      layers=tuple(layers), rms_eps=float(cfg["norm"]["eps"]), bos_token_id=int(cfg.get("bos_token_id", 1)),
+                      eos_token_ids=tuple(eos) if isinstance(eos, list) else (int(eos),), arrangement="sandwich_norm",
+                      norm="layer", embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), tie_embeddings=True)
+
+
 # config.json "architecture" -> parser of a layered hybrid design
 HYBRID_ARCHITECTURES = {"Zadirax": _zadirax_from_config, "Pozalorn": _pozalorn_from_config, "Livitar": _livitar_from_config,
-                        "Gefudra": _gefudra_from_config}
+                        "Gefudra": _gefudra_from_config, "Nigozen": _nigozen_from_config}
 
 
 def _zadirax_preset(name: str, width: int, vocab: int, pairs: int, heads: int, dim: int, ff: int, experts: int,
@@ -446,6 +490,19 @@ def _gefudra_preset(name: str, width: int, vocab: int, groups: int, heads: int, 
     return _gefudra_from_config(cfg, name)
 
 
+def _nigozen_preset(name: str, width: int, vocab: int, heads: int, kv_heads: int, dim: int, vdim: int, rot: int, chunk: int,
+                    ff: int, experts: int, top: int, expert_ff: int, moe_layers: int = 2) -> HybridArch:
+    """Random-init Nigozen models (benchmarks, tests): a layer with a dense feed-forward, then ``moe_layers`` with a
+    mixture of experts."""
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "v_mix": True,
+           "rot": {"base": 500000.0, "dims": rot}, "mask": {"size": chunk}}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top}}
+    cfg = {"width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "embedding": {"scale": 2.0},
+           "layers": [{"type": "attention", "mixer": att, "mlp": {"kind": "dense", "ff": ff}}] +
+                     [{"type": "attention", "mixer": att, "mlp": moe}] * moe_layers}
+    return _nigozen_from_config(cfg, name)
+
+
 HYBRID_PRESETS = {
     # tests / CPU smoke: odd sizes on purpose (nothing a multiple of the MFMA tile)
     "zadirax-tiny": lambda: _zadirax_preset("zadirax-tiny", 96, 300, 2, 3, 24, 136, 5, 2, 40, 56, 40, 8, share=True),
@@ -473,6 +530,13 @@ HYBRID_PRESETS = {
                                                   loop_times=1, wkv_ff=True),
     "gefudra-bench-1536": lambda: _gefudra_preset("gefudra-bench-1536", 1536, 32000, 1, 12, 2, 128, 8960, 512, 768, 1024,
                                                   loop_times=1, wkv_ff=True),
+    # tests / CPU smoke: odd sizes on purpose
+    "nigozen-tiny": lambda: _nigozen_preset("nigozen-tiny", 88, 300, 4, 2, 24, 20, 10, 21, 136, 5, 2, 40),
+    # slices at the layer sizes of real models beside a transformer of equal width (benchmarks/design_compare.py); a
+    # dense feed-forward, and a token's chosen experts together, hold as many weights as the gated dense feed-forward
+    # of the other bench presets
+    "nigozen-bench-1024": lambda: _nigozen_preset("nigozen-bench-1024", 1024, 32000, 8, 2, 128, 128, 64, 1024, 6144, 8, 2, 3072),
+    "nigozen-bench-1536": lambda: _nigozen_preset("nigozen-bench-1536", 1536, 32000, 12, 2, 128, 128, 64, 1024, 13440, 16, 4, 3328),
     # layer sizes of a ~1.5B model (the width, head size, feed-forward and vocabulary of qwen2.5-1.5b)
     "zadirax-1.5b": lambda: _zadirax_preset("zadirax-1.5b", 1536, 151936, 14, 12, 128, 8960, 32, 4, 2240, 512, 768, 64),
 }

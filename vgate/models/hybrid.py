@@ -19,6 +19,11 @@ Layer arrangements (``ARRANGEMENTS``, chosen by ``HybridArch.arrangement``):
                   is the sum of the copies
   pre_norm        x += m * mixer(rmsnorm(x) * w1);  x += m * ff(rmsnorm(x) * w2)   (m = ``residual_mult``; a
                   sublayer's add and the next sublayer's norm are one kernel)
+  sandwich_norm   x += m * norm1b(mixer(norm1(x)));  x += m * norm2b(ff(norm2(x))): a norm before and after each sublayer
+                  (a sublayer's output norm, its add and the next sublayer's norm are one kernel, which for a mixture
+                  of experts also sums a token's weighted expert rows)
+The norms of the last two are RMS or layer norms (``HybridArch.norm``); the embedding rows may be scaled
+(``HybridArch.embed_scale``).
 ``HybridArch.loop`` = (start, stop, times): the layers start .. stop - 1 run ``times`` times in a row with the same
 weights, every pass with caches and states of its own; right before the first layer of each pass the stream
 becomes W_in [x; x0] (``loop.in``, x0 the embedding output).
@@ -37,7 +42,7 @@ from pathlib import Path
 import torch
 
 from vgate.models.config import HybridArch
-from vgate.models.mixers import FEED_FORWARDS, MIXERS, Proj, _f32, _pad8
+from vgate.models.mixers import FEED_FORWARDS, MIXERS, MoEFF, Proj, _f32, _pad8
 from vgate.ops import seq
 from vgate.parallel.comm import TPGroup
 
@@ -239,20 +244,32 @@ class HyperPreNormLayer:
 class PreNormLayer:
     """``pre_norm`` arrangement: x += mult * mixer(rmsnorm(x) * norm1), then x += mult * ff(rmsnorm(x) * norm2)
     (vector weights, fp32 statistics). The residual kernel of a sublayer also makes the normed input of the
-    sublayer that follows (the feed-forward's, or the next layer's first when the model says which that is)."""
+    sublayer that follows (the feed-forward's, or the next layer's first when the model says which that is).
+    ``norm``: "rms" | "layer". POST (:class:`SandwichNormLayer`): each sublayer's output is normed (``norm1b`` /
+    ``norm2b``) before it is added, in the same kernel."""
+    POST = False
 
-    def __init__(self, spec, width: int, eps: float, t: dict, device, f32: bool, mult: float = 1.0):
+    def __init__(self, spec, width: int, eps: float, t: dict, device, f32: bool, mult: float = 1.0, norm: str = "rms"):
         mix = {k[4:]: v for k, v in t.items() if k.startswith("mix.")}
         self.eps, self.mult = eps, float(mult)
+        if norm not in ("rms", "layer"):
+            raise ValueError(f"norm {norm!r}: rms or layer")
+        self.center = norm == "layer"
         if spec.kind == "parallel":
             raise ValueError("the pre_norm arrangement takes single mixers")
         self.mixer = MIXERS[spec.kind](spec.mixer, width, eps, mix, device, f32)
+        self.carries = getattr(self.mixer, "value_mix", False)
         self.norm1 = _f32(t["norm1"], device)
-        self.ff = self.norm2 = None
+        self.norm1b = _f32(t["norm1b"], device) if self.POST else None
+        self.ff = self.norm2 = self.norm2b = None
+        self.ff_kw = {"out_f32": True}
         if spec.mlp:
             mlp = {k[4:]: v for k, v in t.items() if k.startswith("mlp.")}
             self.ff = FEED_FORWARDS[spec.mlp["kind"]](spec.mlp, width, mlp, device, f32)
             self.norm2 = _f32(t["norm2"], device)
+            self.norm2b = _f32(t["norm2b"], device) if self.POST else None
+            if isinstance(self.ff, MoEFF) and self.ff.shared is None:
+                self.ff_kw["combine"] = False   # the residual kernel sums a token's expert rows
         self.proj, self.col = _fuse_inputs(self.mixer, [], width, device, f32)
 
     @staticmethod
@@ -275,27 +292,44 @@ class PreNormLayer:
         """st.x: the fp32 stream; st.h: the normed input in the activation dtype (``st.h_ready``: the kernel before
         has made this layer's already); st.next_norm: the norm weight of the layer that follows, or None."""
         if not st.h_ready:
-            seq.norm_rows(st.x, self.norm1, self.eps, st.h)
+            seq.norm_rows(st.x, self.norm1, self.eps, st.h, center=self.center)
         P = self.proj(st.h) if self.proj is not None else None
-        y = self.mixer.forward(st.h, P, self.cols, sv, cache)
+        y = self.mixer.forward(st.h, P, self.cols, sv, cache, **({"carry": st.carry} if self.carries else {}))
+        post = self.norm1b
         if self.ff is not None:
-            seq.residual_norm(st.x, y, self.mult, self.norm2, self.eps, st.h)
-            y = self.ff.forward(st.h, out_f32=True)
-        seq.residual_norm(st.x, y, self.mult, st.next_norm, self.eps, st.h if st.next_norm is not None else None)
+            seq.residual_norm(st.x, y, self.mult, self.norm2, self.eps, st.h, post_w=post, center=self.center)
+            y, post = self.ff.forward(st.h, **self.ff_kw), self.norm2b
+        seq.residual_norm(st.x, y, self.mult, st.next_norm, self.eps, st.h if st.next_norm is not None else None,
+                          post_w=post, center=self.center)
         st.h_ready = st.next_norm is not None
 
 
+class SandwichNormLayer(PreNormLayer):
+    """``sandwich_norm`` arrangement: x += mult * norm1b(mixer(norm1(x))), then x += mult * norm2b(ff(norm2(x)))."""
+    POST = True
+
+    @staticmethod
+    def shapes(spec, width: int) -> dict:
+        out = PreNormLayer.shapes(spec, width)
+        out["norm1b"] = (width,)
+        if spec.mlp:
+            out["norm2b"] = (width,)
+        return out
+
+
 class _PreStream:
-    """The stream of one ``pre_norm`` step: ``x`` fp32 [T, W], ``h`` the next sublayer's normed input."""
+    """The stream of one ``pre_norm`` or ``sandwich_norm`` step: ``x`` fp32 [T, W], ``h`` the next sublayer's normed
+    input, ``carry`` what the mixers of the step's layer runs hand on to each other."""
 
     def __init__(self, T: int, W: int, act_dtype, device):
         self.x = torch.empty(T, W, dtype=torch.float32, device=device)
         self.h = torch.empty(T, W, dtype=act_dtype, device=device)
         self.h_ready, self.next_norm = False, None
+        self.carry: dict = {}
 
 
 ARRANGEMENTS = {"gated_parallel": GatedParallelLayer, "post_norm": PostNormLayer, "hyper_pre_norm": HyperPreNormLayer,
-                "pre_norm": PreNormLayer}
+                "pre_norm": PreNormLayer, "sandwich_norm": SandwichNormLayer}
 
 
 class _HyperStream:
@@ -372,7 +406,10 @@ class HybridModel:
         tensors = load_tensors(arch, weights_path) if weights_path else random_tensors(arch, seed)
         self.embed = tensors["embed"].to(self.device, self.act_dtype).contiguous()
         layer_cls = ARRANGEMENTS[arch.arrangement]
-        extra = {"mult": arch.residual_mult} if arch.arrangement == "pre_norm" else {}
+        self.pre = arch.arrangement in ("pre_norm", "sandwich_norm")
+        extra = {"mult": arch.residual_mult, "norm": arch.norm} if self.pre else {}
+        if not self.pre and (arch.norm != "rms" or arch.embed_scale != 1.0):
+            raise ValueError(f"layer norms and scaled embeddings need the pre_norm or sandwich_norm arrangement, not {arch.arrangement}")
         owned: dict = {}
         self.layers: list = []        # one entry per layer RUN (a looped layer once per pass): caches are per run
         self.pass_start: list = []    # whether a pass of the loop starts at that run
@@ -387,6 +424,10 @@ class HybridModel:
                 raise ValueError(f"layer {i} shares weights with layer {j} of another mixer type")
             self.layers.append(owned[j])
             self.pass_start.append(first)
+        if any(getattr(L, "carries", False) != getattr(L.mixer, "value_mix", False) for L in owned.values()):
+            raise ValueError("mixed values need the pre_norm or sandwich_norm arrangement")
+        if len({L.mixer.G * L.mixer.V for L in owned.values() if getattr(L.mixer, "value_mix", False)}) > 1:
+            raise ValueError("layers that mix values need the same kv_heads * vdim")
         self._owned = owned
         self.loop_in = Proj(tensors["loop.in"], self.device, self.f32) if arch.loop is not None else None
         # depth-average coefficients belong to the position in the stack, not to the (possibly shared) weights
@@ -422,7 +463,7 @@ class HybridModel:
     def forward(self, sv, caches, part_size: int = 0, return_hidden: bool = False) -> torch.Tensor:
         """One step. Returns fp32 logits [S, vocab] of the sample rows, or with ``return_hidden`` the
         fp32 residual stream [T, width] after the last layer."""
-        if self.hyper or self.arch.arrangement == "pre_norm":
+        if self.hyper or self.pre:
             x = self._forward_hyper(sv, caches) if self.hyper else self._forward_pre(sv, caches)
             return x if return_hidden else self._padded_logits(x, sv)
         T = sv.T
@@ -464,10 +505,11 @@ class HybridModel:
         return st.x
 
     def _forward_pre(self, sv, caches) -> torch.Tensor:
-        """The layer loop of the ``pre_norm`` arrangement, with the looped stretch; returns the fp32 stream."""
+        """The layer loop of the ``pre_norm`` and ``sandwich_norm`` arrangements, with the looped stretch; returns the
+        fp32 stream."""
         T, W = sv.T, self.arch.hidden_size
         st = _PreStream(T, W, self.act_dtype, self.device)
-        seq.embed_rows(sv.ids, self.embed, st.x, prev=sv.prev_tokens)
+        seq.embed_rows(sv.ids, self.embed, st.x, prev=sv.prev_tokens, scale=self.arch.embed_scale)
         x0 = pair = None
         if self.loop_in is not None:
             x0 = st.x.clone()
@@ -503,7 +545,8 @@ class HybridModel:
             n = self.final_norm
             seq.tanh_norm_rows(x, n.alpha, n.w, n.b, hn, rows=rows)
         else:
-            seq.norm_rows(x, self.final_norm, self.arch.rms_eps, hn, rows=rows, scalar=self.scalar_norm)
+            seq.norm_rows(x, self.final_norm, self.arch.rms_eps, hn, rows=rows, scalar=self.scalar_norm,
+                          center=self.arch.norm == "layer")
         return self.head(hn, out_f32=True, out=out)[:, : self.arch.vocab_size]
 
 
@@ -584,7 +627,9 @@ def random_tensors(arch: HybridArch, seed: int = 0) -> dict:
         elif len(shape) == 2:
             std = 0.5 if name == "embed" else 1.0 / math.sqrt(shape[1])
             w = torch.randn(shape, generator=g) * std
-        elif leaf in ("norm", "norm1", "norm2") or name == "final.norm":
+        elif leaf == "vmix":             # a blend weight between two layers' values
+            w = 0.2 + 0.6 * torch.rand(shape, generator=g)
+        elif leaf in ("norm", "norm1", "norm2", "norm1b", "norm2b") or name == "final.norm":
             w = 1.0 + 0.1 * torch.randn(shape, generator=g)
         else:
             w = 0.3 * torch.randn(shape, generator=g)

@@ -14,7 +14,8 @@ spec, so another design can reuse a mixer with other values.
   cache, optionally with one mean key / value per block of tokens that has left the window, a sink in the
   softmax denominator, query / key norms over the head or the whole projection, values rotated by
   their position, a bias on the scores that depends on the distance (logarithmic penalty or a learned
-  table over distance buckets), per-head and per-position query temperatures, a sigmoid output gate.
+  table over distance buckets), per-head and per-position query temperatures, a sigmoid output gate; chunks
+  of positions instead of a window; values blended with an earlier layer's values of the same token.
 * :class:`LinearAttention` — decayed outer-product recurrence S <- diag(a) S + k v^T, o = S^T q over an
   fp32 state per head in a state slot; the decay is a constant per head or a gated value per key channel;
   optional rotary positions on q / k.
@@ -22,8 +23,9 @@ spec, so another design can reuse a mixer with other values.
   current token's own outer product, a decay exp(-exp(.)) per key channel from a low-rank gate, and every
   projection reading its own blend of the token's and the previous token's input (which is part of the state).
 * :class:`ParallelMixers` — two mixers reading the same input, their outputs added with fixed scales.
-* :class:`DenseFF`, :class:`MoEFF` — gated feed-forward; mixture of gated experts (sigmoid scores with a
-  selection-only correction or softmax scores, clamped or SiLU experts, optional shared expert).
+* :class:`DenseFF`, :class:`MoEFF` — feed-forward (gated pair, or one matrix and an activation); mixture of such
+  experts (sigmoid scores with a selection-only correction, softmax scores over all experts or over the chosen,
+  optional shared expert).
 """
 from __future__ import annotations
 
@@ -80,8 +82,9 @@ class Proj:
             if out is None:
                 out = torch.empty(M, self.out_features, dtype=torch.bfloat16, device=x.device)
             return seq.glu_rows(ops.linear(x, self.lin), out, self.pair_act, limit=self.limit, alpha=self.alpha)
-        if self.packed and act == 0:
-            return ops.linear(x, self.lin, out=out, out_f32=out_f32)
+        if self.packed:   # (a single matrix's activation is a row kernel behind the packed GEMM)
+            y = ops.linear(x, self.lin, out=out, out_f32=out_f32)
+            return seq.act_rows(y, act) if act else y
         dt = torch.float32 if (out_f32 or self.f32) else torch.bfloat16
         if out is None:
             out = torch.empty(M, self.out_features, dtype=dt, device=x.device)
@@ -280,6 +283,11 @@ class WindowAttention:
     (:func:`distance_buckets`). ``gate`` "sigmoid": the heads' outputs are multiplied by sigmoid(W_g h)
     before the output projection. ``rot.layout`` "pairs" (entry 2i with 2i + 1, the default) or "half" (entry i
     with i + dims / 2). ``softcap`` c > 0: the scaled score s becomes c tanh(s / c).
+    ``chunk`` c > 0: position i sees only the j <= i of its own chunk, floor(j / c) = floor(i / c), counted from the
+    sequence's position 0 (beside ``window``; not with pooled blocks). ``sink`` "one": a sink whose logit is 0 (one is
+    added to the softmax denominator), without a tensor. ``value_mix``: in every layer run with it but a step's
+    first, the values become (1 - lam) v + lam v_first before they are cached, lam the tensor ``vmix`` and v_first that
+    first run's values of the same token (all such layers need the same kv_heads * vdim).
     ``maps`` {count: 2, init: d}: every head has two query / key maps (q and k carry [map 1, map 2] per head,
     each of size dim) that are two attentions over the same values; with lam = exp(lq1 . lk1) - exp(lq2 . lk2) + d
     (tensors ``lq1`` .. ``lk2`` [dim], one number per layer) the head's output is (a1 - lam a2), divided by its
@@ -300,6 +308,11 @@ class WindowAttention:
         self.window = self.FULL if m.get("window") is None else int(m["window"])
         if self.window < 1 or self.pool < 0 or self.window > self.FULL:
             raise ValueError("window_attention: window >= 1, pool >= 0")
+        self.chunk = int(m.get("chunk") or 0)
+        if not 0 <= self.chunk <= self.FULL or (self.chunk and self.pool):
+            raise ValueError("window_attention: chunk >= 1 (or none), not with pooled blocks")
+        self.value_mix = bool(m.get("value_mix"))
+        self.lam_v = float(tensors["vmix"].float().reshape(())) if self.value_mix else 0.0
         if self.pool and m.get("window") is None:
             raise ValueError("window_attention: pooled blocks need a window")
         self.qk_norm = m.get("qk_norm", "none")
@@ -361,7 +374,9 @@ class WindowAttention:
                 self.qw = torch.ones(self.D if per_head else self.HQ * self.D, dtype=torch.float32, device=dev)
                 self.kw = torch.ones(self.D if per_head else self.GK * self.D, dtype=torch.float32, device=dev)
         self.sink = None
-        if m.get("sink"):   # (with two maps: the head's sink in both)
+        if m.get("sink") == "one":
+            self.sink = torch.zeros(self.HQ, dtype=torch.float32, device=dev)
+        elif m.get("sink"):   # (with two maps: the head's sink in both)
             sk = tensors["sink"]
             self.sink = _f32(regroup(sk.repeat_interleave(2)) if self.maps == 2 else sk, dev)
         self.head_temp = _f32(tensors["temp"], dev) if m.get("head_temp") else None
@@ -409,8 +424,10 @@ class WindowAttention:
             out.update({"r1": (H,), "r2": (H,)})
         elif kind == "table":   # None: the number of buckets, which only the tensor gives
             out["rel"] = (None, H)
-        if spec.get("sink"):
+        if spec.get("sink") and spec["sink"] != "one":
             out["sink"] = (H,)
+        if spec.get("value_mix"):
+            out["vmix"] = ()
         if spec.get("out_bias"):
             out["o.b"] = (width,)
         return out
@@ -439,14 +456,20 @@ class WindowAttention:
     def nbytes(self) -> int:
         return self.o.nbytes()
 
-    def forward(self, h, P, cols, sv, cache) -> torch.Tensor:
+    def forward(self, h, P, cols, sv, cache, carry: dict | None = None) -> torch.Tensor:
+        """``carry``: what the layer runs of one step hand on to each other (needed with ``value_mix``)."""
         T = h.shape[0]
         kc, vc, kp, vp, vt = cache
         q = torch.empty(T, self.HQ * self.D, dtype=h.dtype, device=h.device)
-        seq.window_write(cols(P, "q"), cols(P, "k"), cols(P, "v"), self.qw, self.kw, self.eps, self.qk_norm == "all",
+        v, v_first = cols(P, "v"), None
+        if self.value_mix:
+            v_first = carry.get("values")
+            if v_first is None:   # (a view of this layer's fused projection, which it keeps alive for the step)
+                carry["values"] = v
+        seq.window_write(cols(P, "q"), cols(P, "k"), v, self.qw, self.kw, self.eps, self.qk_norm == "all",
                          sv.positions, sv.slots, self.inv_freq, self.rot_dims, self.v_freq, kc, vc, q, self.HQ, self.GK, vt=vt,
                          q_head_scale=self.head_temp, q_temp_coef=self.q_temp[0], q_temp_every=self.q_temp[1],
-                         rot_half=self.rot_half)
+                         rot_half=self.rot_half, v_other=v_first, lam=self.lam_v)
         if self.pool:
             seq.window_pool(kc, vc, kp, vp, sv.positions, sv.block_tables, sv.query_start, self.pool,
                             num_seqs=sv.num_seqs or None)
@@ -455,7 +478,7 @@ class WindowAttention:
         seq.window_attn(q, kc, vc, kp, vp, sv.block_tables, sv.context_lens, sv.query_start, o, self.scale, self.HQ,
                         self.window, self.pool, self.sink, self.v_freq, num_seqs=sv.num_seqs or None, vt=vt,
                         bias_kind=self.bias_kind, bias_a=self.bias_a, bias_b=self.bias_b,
-                        gate=gate if self.maps == 1 else None, softcap=self.softcap)
+                        gate=gate if self.maps == 1 else None, softcap=self.softcap, chunk=self.chunk)
         if self.maps == 2:   # (a1 - lam a2) / rms * (1 - init) * sigmoid(gate), heads back in their own order
             both, o = o, torch.empty(T, self.H * self.V, dtype=h.dtype, device=h.device)
             seq.map_pair_combine(both, self.lam, self.out_scale, self.eps, gate, o, self.H, self.G, self.V)
@@ -671,45 +694,62 @@ MIXERS = {c.kind: c for c in (LatentAttention, GeneralDelta, WindowAttention, Li
 # ------------------------------------------------------------------------------------ feed-forwards
 class DenseFF:
     """down(act(gate h) * (up h)); spec ``act``: "silu" (default), "gelu_tanh", or "clamped" with ``limit`` L:
-    g = min(gate h, L), u = clamp(up h, -L, L), down(g * sigmoid(ALPHA g) * (u + 1))."""
+    g = min(gate h, L), u = clamp(up h, -L, L), down(g * sigmoid(ALPHA g) * (u + 1)). ``gated`` False (no gate matrix):
+    down(act(up h)) with act "gelu" (erf form) or "relu2" (max(., 0)^2)."""
     ACTS = {"silu": seq.ACT_SILU_MUL, "gelu_tanh": seq.ACT_GELU_TANH_MUL, "clamped": seq.ACT_CLAMPED_GLU}
+    PLAIN_ACTS = {"gelu": seq.ACT_GELU, "relu2": seq.ACT_RELU2}
     ALPHA = 1.702
 
     def __init__(self, spec: dict, width: int, tensors: dict, device, f32: bool):
+        self.gated = bool(spec.get("gated", True))
         act = spec.get("act", "silu")
-        if act not in self.ACTS:
-            raise ValueError(f"dense feed-forward: act {act!r}")
+        if act not in (self.ACTS if self.gated else self.PLAIN_ACTS):
+            raise ValueError(f"dense feed-forward: act {act!r} ({'gated' if self.gated else 'without a gate'})")
+        if not self.gated:
+            self.act = self.PLAIN_ACTS[act]
+            self.up, self.down = Proj(tensors["up"], device, f32), Proj(tensors["down"], device, f32)
+            return
         self.gate_up = Proj(torch.cat([tensors["gate"], tensors["up"]]), device, f32, silu_pair=True,
                             pair_act=self.ACTS[act], limit=float(spec.get("limit", 0.0)), alpha=self.ALPHA)
         self.down = Proj(tensors["down"], device, f32)
 
     @staticmethod
     def shapes(spec: dict, width: int) -> dict:
-        return {"gate": (spec["ff"], width), "up": (spec["ff"], width), "down": (width, spec["ff"])}
+        out = {"gate": (spec["ff"], width)} if spec.get("gated", True) else {}
+        out.update({"up": (spec["ff"], width), "down": (width, spec["ff"])})
+        return out
 
     def nbytes(self) -> int:
-        return self.gate_up.nbytes() + self.down.nbytes()
+        return (self.gate_up if self.gated else self.up).nbytes() + self.down.nbytes()
 
     def forward(self, h: torch.Tensor, out_f32: bool = False) -> torch.Tensor:
-        return self.down(self.gate_up(h), out_f32=out_f32)
+        return self.down(self.gate_up(h) if self.gated else self.up(h, act=self.act), out_f32=out_f32)
 
 
 class MoEFF:
-    """Routed experts: scores s = sigmoid(z) or softmax(z) over all experts (``router.score``, fp32); the
+    """Routed experts: scores s = sigmoid(z), softmax(z) over all experts or "top_softmax", the softmax over the
+    chosen logits alone (``router.score``, fp32); the
     ``top`` largest of s (+ a selection-only ``correction`` tensor unless ``router.correction`` is False)
     are chosen, weighted by their scores over the chosen scores' sum, times ``router.scale``. Expert
     (``expert.act``): "clamped": g = min(gate h, L), u = clamp(up h, -L, L), down(g * sigmoid(alpha g) * (u + 1));
-    "silu": down(silu(gate h) * (up h)). ``shared`` {ff}: a dense gated expert every token runs, added."""
+    "silu": down(silu(gate h) * (up h)); without a gate matrix (``expert.gated`` False) down(act(up h)) with act "gelu"
+    or "relu2". ``shared`` {ff}: a dense gated expert every token runs, added."""
     ALPHA = 1.702
     SUM_EPS = 1e-20
+    SCORES = {"sigmoid": seq.ROUTE_SIGMOID, "softmax": seq.ROUTE_SOFTMAX, "top_softmax": seq.ROUTE_TOP_SOFTMAX}
 
     def __init__(self, spec: dict, width: int, tensors: dict, device, f32: bool):
         r = spec["router"]
         self.E, self.top = int(r["experts"]), int(r["top"])
         self.ff = int(spec["expert"]["ff"])
-        self.act = {"clamped": seq.ACT_CLAMPED_GLU, "silu": seq.ACT_SILU_MUL}[spec["expert"].get("act", "clamped")]
+        self.gated = bool(spec["expert"].get("gated", True))
+        acts = {"clamped": seq.ACT_CLAMPED_GLU, "silu": seq.ACT_SILU_MUL} if self.gated else DenseFF.PLAIN_ACTS
+        self.act = acts[spec["expert"].get("act", "clamped")]
         self.limit = float(spec["expert"]["limit"]) if self.act == seq.ACT_CLAMPED_GLU else 0.0
-        self.softmax = {"sigmoid": False, "softmax": True}[r.get("score", "sigmoid")]
+        self.score = self.SCORES[r.get("score", "sigmoid")]
+        if not 1 <= self.top <= self.E:
+            raise ValueError("moe feed-forward: 1 <= router.top <= router.experts")
+        self.sum_eps = 0.0 if self.score == seq.ROUTE_TOP_SOFTMAX else self.SUM_EPS
         self.scale = float(r.get("scale", 1.0))
         dev = torch.device(device)
         dt = torch.float32 if f32 else torch.bfloat16
@@ -717,7 +757,8 @@ class MoEFF:
         self.router = Proj(tensors["router"], dev, f32, allow_packed=False)  # fp32 logits, N = experts
         self.corr = _f32(tensors["correction"], dev) if r.get("correction", True) else None
         st = lambda n: torch.stack([tensors[f"e{e}.{n}"] for e in range(self.E)]).to(dev, dt).contiguous()  # noqa: E731
-        self.gate, self.up, self.down = st("gate"), st("up"), st("down")
+        self.gate = st("gate") if self.gated else None
+        self.up, self.down = st("up"), st("down")
         self.shared = None
         if spec.get("shared"):
             sh = {k[len("shared."):]: v for k, v in tensors.items() if k.startswith("shared.")}
@@ -730,31 +771,40 @@ class MoEFF:
         if spec["router"].get("correction", True):
             out["correction"] = (E,)
         for e in range(E):
-            out.update({f"e{e}.gate": (ff, width), f"e{e}.up": (ff, width), f"e{e}.down": (width, ff)})
+            if spec["expert"].get("gated", True):
+                out[f"e{e}.gate"] = (ff, width)
+            out.update({f"e{e}.up": (ff, width), f"e{e}.down": (width, ff)})
         if spec.get("shared"):
             out.update({"shared." + k: v for k, v in DenseFF.shapes(spec["shared"], width).items()})
         return out
 
     def nbytes(self) -> int:
-        return (self.router.nbytes() + 3 * self.gate.numel() * self.gate.element_size()
+        return (self.router.nbytes() + (3 if self.gated else 2) * self.up.numel() * self.up.element_size()
                 + (self.shared.nbytes() if self.shared else 0))
 
-    def forward(self, h: torch.Tensor, out_f32: bool = False) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, out_f32: bool = False, combine: bool = True):
+        """``combine`` False (no shared expert): the tuple (expert rows, pos, wts) for a kernel that sums a token's
+        weighted rows itself (:func:`vgate.ops.seq.residual_norm`)."""
         T, W = h.shape
         dev, dt = h.device, h.dtype
         z = self.router(h, out_f32=True)
         idx = torch.empty(T, self.top, dtype=torch.int32, device=dev)
         wts = torch.empty(T, self.top, dtype=torch.float32, device=dev)
-        seq.moe_route(z, self.corr, self.top, self.SUM_EPS, idx, wts, softmax=self.softmax, scale=self.scale)
+        seq.moe_route(z, self.corr, self.top, self.sum_eps, idx, wts, score=self.score, scale=self.scale)
         rows = torch.empty(T * self.top, dtype=torch.int32, device=dev)
         pos = torch.empty(T * self.top, dtype=torch.int32, device=dev)
         off = torch.empty(self.E + 1, dtype=torch.int32, device=dev)
         seq.moe_sort(idx, self.E, rows, pos, off)
         a1 = torch.empty(T * self.top, self.ff, dtype=dt, device=dev)
-        seq.gemm(h, self.gate, a1, w2=self.up, a_rows=rows, group_off=off, act=self.act, limit=self.limit,
-                 alpha=self.ALPHA)
+        if self.gated:
+            seq.gemm(h, self.gate, a1, w2=self.up, a_rows=rows, group_off=off, act=self.act, limit=self.limit,
+                     alpha=self.ALPHA)
+        else:
+            seq.gemm(h, self.up, a1, a_rows=rows, group_off=off, act=self.act)
         y = torch.empty(T * self.top, W, dtype=dt, device=dev)
         seq.gemm(a1, self.down, y, group_off=off)
+        if not combine and self.shared is None:
+            return y, pos, wts
         out = torch.empty(T, W, dtype=torch.float32 if out_f32 else dt, device=dev)
         seq.moe_combine(y, pos, wts, out, add=self.shared.forward(h, out_f32=out_f32) if self.shared else None)
         return out

@@ -42,7 +42,8 @@ def _C():
     return _Traced(mod) if _TRACE else mod
 
 
-ACT_NONE, ACT_SILU_MUL, ACT_CLAMPED_GLU, ACT_TANH, ACT_GELU_TANH_MUL = 0, 1, 2, 3, 4
+ACT_NONE, ACT_SILU_MUL, ACT_CLAMPED_GLU, ACT_TANH, ACT_GELU_TANH_MUL, ACT_GELU, ACT_RELU2 = 0, 1, 2, 3, 4, 5, 6
+ROUTE_SIGMOID, ROUTE_SOFTMAX, ROUTE_TOP_SOFTMAX = 0, 1, 2   # what a router chooses and weighs by (see moe_route)
 BIAS_NONE, BIAS_LOG, BIAS_TABLE = 0, 1, 2   # distance term of an attention score (see window_attn)
 MAX_STREAMS = 16            # copies of the residual stream hyper_mix takes
 WINDOW_SPLIT = os.environ.get("VGATE_WINDOW_SPLIT", "1") == "1"   # "0": one workgroup per decoded 16-row tile
@@ -61,6 +62,10 @@ def _act(g: torch.Tensor, u: torch.Tensor | None, act: int, limit: float, alpha:
         return torch.tanh(g)
     if act == ACT_GELU_TANH_MUL:
         return 0.5 * g * (1.0 + torch.tanh(0.7978845608028654 * (g + 0.044715 * g * g * g))) * u
+    if act == ACT_GELU:
+        return 0.5 * g * (1.0 + torch.erf(g * 0.7071067811865476))
+    if act == ACT_RELU2:
+        return g.clamp(min=0.0).square()
     return g
 
 
@@ -100,27 +105,35 @@ def gemm(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, w2: torch.Tensor |
     return out
 
 
+def _normed(x: torch.Tensor, eps: float, center: bool) -> torch.Tensor:
+    """x / sqrt(mean(x^2) + eps) over the last axis, after the mean is taken off if ``center`` (a layer norm)."""
+    if center:
+        x = x - x.mean(-1, keepdim=True)
+    return x * (1.0 / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps))
+
+
 def norm_rows(x: torch.Tensor, w: torch.Tensor, eps: float, out: torch.Tensor, rows: torch.Tensor | None = None,
-              scalar: bool = False) -> torch.Tensor:
-    """out[m] = x[rows[m]] / sqrt(mean(x^2) + eps) * w (w fp32: one number if ``scalar``)."""
+              scalar: bool = False, center: bool = False) -> torch.Tensor:
+    """out[m] = x[rows[m]] / sqrt(mean(x^2) + eps) * w (w fp32: one number if ``scalar``); ``center``: a layer norm
+    (the row's mean is taken off first)."""
     if x.is_cuda:
-        _C().norm_rows(x, w, eps, out, rows, scalar)
+        _C().norm_rows(x, w, eps, out, rows, scalar, center)
         return out
     xf = x.float()
     xf = xf[rows.long()] if rows is not None else xf[: out.shape[0]]
-    y = xf * (1.0 / torch.sqrt(xf.pow(2).mean(-1, keepdim=True) + eps)) * w
-    out.copy_(y)
+    out.copy_(_normed(xf, eps, center) * w)
     return out
 
 
-def embed_rows(ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor, prev: torch.Tensor | None = None) -> torch.Tensor:
-    """fp32 rows of the embedding table; ids < 0 name the previous step's sample prev[-id - 1]."""
+def embed_rows(ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor, prev: torch.Tensor | None = None,
+               scale: float = 1.0) -> torch.Tensor:
+    """fp32 rows of the embedding table times ``scale``; ids < 0 name the previous step's sample prev[-id - 1]."""
     if table.is_cuda:
-        _C().embed_rows(ids, table, out, prev)
+        _C().embed_rows(ids, table, out, prev, scale)
         return out
     if prev is not None and bool((ids < 0).any()):
         ids = torch.where(ids < 0, prev.to(ids.device)[(-ids - 1).clamp(min=0).long()], ids)
-    out.copy_(table[ids.long()].float())
+    out.copy_(table[ids.long()].float() * scale)
     return out
 
 
@@ -292,14 +305,19 @@ def delta_rule(r, k, v, g, a, wl, w0, ab, nw, state, state_slots, context_lens, 
         state[slot] = St
 
 
-def moe_route(z, corr, top: int, norm_eps: float, idx, wts, softmax: bool = False, scale: float = 1.0) -> None:
+def moe_route(z, corr, top: int, norm_eps: float, idx, wts, score: int = ROUTE_SIGMOID, scale: float = 1.0) -> None:
     """idx / wts [T, top]: the ``top`` largest of s + corr with s = sigmoid(z), or softmax(z) over all
-    experts; weights s of the chosen over (their sum + norm_eps), times ``scale``."""
+    experts (``score``); weights s of the chosen over (their sum + norm_eps), times ``scale``. ROUTE_TOP_SOFTMAX: the
+    ``top`` largest of z + corr, weighted by the softmax of z over the chosen alone (norm_eps 0), times ``scale``."""
     if z.is_cuda:
-        _C().moe_route(z, corr, top, norm_eps, idx, wts, softmax, scale)
+        _C().moe_route(z, corr, top, norm_eps, idx, wts, score, scale)
         return
-    s = torch.softmax(z, -1) if softmax else torch.sigmoid(z)
-    choice = s + corr if corr is not None else s
+    if score == ROUTE_TOP_SOFTMAX:
+        s, choice = torch.exp(z - z.amax(-1, keepdim=True)), z
+    else:
+        s = torch.softmax(z, -1) if score == ROUTE_SOFTMAX else torch.sigmoid(z)
+        choice = s
+    choice = choice + corr if corr is not None else choice
     # arg-max rounds, lowest index first on ties (the kernel's order)
     c = choice.clone()
     picks = []
@@ -397,18 +415,36 @@ def glu_rows(gu: torch.Tensor, out: torch.Tensor, act: int, limit: float = 0.0, 
     return out
 
 
-def residual_norm(x: torch.Tensor, y: torch.Tensor, mult: float, w: torch.Tensor | None = None, eps: float = 0.0,
-                  h_out: torch.Tensor | None = None) -> None:
-    """x += mult * y in fp32 (x fp32 [T, W], y fp32 or the activation dtype). With ``w`` [W]: also
-    h_out = x / sqrt(mean(x^2) + eps) * w from the new x, rounded to h_out's dtype."""
+def act_rows(x: torch.Tensor, act: int, out: torch.Tensor | None = None) -> torch.Tensor:
+    """act(x) over bf16 rows (ACT_TANH, ACT_GELU, ACT_RELU2), in place unless ``out`` is given."""
+    out = x if out is None else out
     if x.is_cuda:
-        _C().residual_norm(x, y, mult, w, eps, h_out)
+        _C().act_rows(x, out, act)
+        return out
+    out.copy_(_act(x[: out.shape[0]].float(), None, act, 0.0, 0.0))
+    return out
+
+
+def residual_norm(x: torch.Tensor, y, mult: float, w: torch.Tensor | None = None, eps: float = 0.0,
+                  h_out: torch.Tensor | None = None, post_w: torch.Tensor | None = None, center: bool = False) -> None:
+    """x += mult * u in fp32 (x fp32 [T, W]). u is ``y`` (fp32 or the activation dtype), or with ``y`` a tuple (rows
+    [T * top, W], pos, wts [T, top]) a token's weighted expert rows (see :func:`moe_combine`); with ``post_w`` [W]:
+    u = norm(.) * post_w. With ``w`` [W]: also h_out = norm(x) * w from the new x, rounded to h_out's dtype.
+    norm: division by sqrt(mean(.^2) + eps), after the mean is taken off if ``center`` (a layer norm)."""
+    pos = wts = None
+    if isinstance(y, tuple):
+        y, pos, wts = y
+    if x.is_cuda:
+        _C().residual_norm(x, y, mult, w, eps, h_out, post_w, center, pos, wts)
         return
-    T = y.shape[0]
-    x[:T] += mult * y.float()
+    u = y.float()
+    if wts is not None:
+        u = (u[pos.view(wts.shape).long()] * wts[:, :, None]).sum(1)
+    if post_w is not None:
+        u = _normed(u, eps, center) * post_w
+    x[: u.shape[0]] += mult * u
     if w is not None:
-        xf = x[: h_out.shape[0]]
-        h_out.copy_(xf * (1.0 / torch.sqrt(xf.pow(2).mean(-1, keepdim=True) + eps)) * w)
+        h_out.copy_(_normed(x[: h_out.shape[0]], eps, center) * w)
 
 
 def pair_rows(a: torch.Tensor, b: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
@@ -495,7 +531,7 @@ def _rope_pairs_heads(x: torch.Tensor, pos: torch.Tensor, inv_freq: torch.Tensor
 
 def window_write(q, k, v, qw, kw, eps: float, norm_all: bool, positions, slots, inv_freq, rot_dims: int, v_freq,
                  kc, vc, q_out, H: int, G: int, vt=None, q_head_scale=None, q_temp_coef: float = 0.0,
-                 q_temp_every: int = 1, rot_half: bool = False) -> None:
+                 q_temp_every: int = 1, rot_half: bool = False, v_other=None, lam: float = 0.0) -> None:
     """Prepare one step's queries, keys and values of a window-attention layer.
     q [T, H * D], k [T, G * D], v [T, G * V] (biases already added). Query / key RMS norm (``qw`` / ``kw``
     None: none; ``norm_all``: over the whole projection with a [heads * D] weight, else per head with a
@@ -506,14 +542,17 @@ def window_write(q, k, v, qw, kw, eps: float, norm_all: bool, positions, slots, 
     ``vt`` (GPU, bf16): a second copy of the values laid out [pages, G, V, page], the operand layout of
     the MFMA attention kernel's weighted sum. ``rot_half``: entry i is paired with entry i + rot_dims / 2 instead
     of 2i with 2i + 1. The value cache may have fewer heads than the key cache (vc.shape[1] divides G: consecutive
-    key heads share a value head); v then is [T, value heads * V]."""
+    key heads share a value head); v then is [T, value heads * V]. ``v_other`` (rows like v's): the values become
+    (1 - lam) v + lam v_other in fp32 before anything else happens to them."""
     if q.is_cuda:
         _C().window_write(q, k, v, qw, kw, eps, norm_all, positions, slots, inv_freq, rot_dims, v_freq, kc, vc, q_out, H, G, vt,
-                          q_head_scale, q_temp_coef, q_temp_every, rot_half)
+                          q_head_scale, q_temp_coef, q_temp_every, rot_half, v_other, lam)
         return
     T = q.shape[0]
     D, V, page = kc.shape[3], vc.shape[3], kc.shape[2]
     qf, kf, vf = q.float(), k.float(), v.float()
+    if v_other is not None:
+        vf = (1.0 - lam) * vf + lam * v_other[:T].float()
 
     def norm(x, w, heads):
         if w is None:
@@ -568,7 +607,8 @@ def window_pool(kc, vc, kp, vp, positions, block_tables, query_start, pool: int,
 
 def window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out, scale: float, H: int, window: int,
                 pool: int, sink, v_freq, num_seqs: int | None = None, vt=None, prefill_kernel: int = 0,
-                bias_kind: int = BIAS_NONE, bias_a=None, bias_b=None, gate=None, softcap: float = 0.0) -> None:
+                bias_kind: int = BIAS_NONE, bias_a=None, bias_b=None, gate=None, softcap: float = 0.0,
+                chunk: int = 0) -> None:
     """out[t, h] = sum_j p_j value_j over the keys position i of token t sees: the tokens j with
     0 <= i - j < window and, with ``pool`` = P > 0, the pooled row of every block b with
     b P + P - 1 <= i - window; p = softmax(scale q . key) over both kinds together, with exp(sink[h]) added
@@ -580,16 +620,17 @@ def window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out,
     the MFMA kernels (``prefill_kernel``: which one prompt portions take, 0 = tiles staged in LDS for 64 rows,
     1 = 16 rows per workgroup with the tiles shared out over its waves). ``softcap`` c > 0: the scaled score s
     becomes c tanh(s / c) (not together with a distance term). The value caches may have fewer heads than the key
-    cache (consecutive key heads share a value head)."""
+    cache (consecutive key heads share a value head). ``chunk`` c > 0: of those keys only the ones with
+    floor(j / c) = floor(i / c) are seen (positions counted from the sequence's first; not with pooled blocks)."""
     if q.is_cuda:
         parts, scratch = 1, None
         if vt is not None and WINDOW_SPLIT:   # decoded tokens of the MFMA kernel: several workgroups per 16-row tile
             parts, n = _C().window_attn_split(q.shape[0], block_tables.shape[0], H, kc.shape[1], kc.shape[3], vc.shape[3],
-                                              kc.dtype == torch.float32, kc.shape[2])
+                                              kc.dtype == torch.float32, kc.shape[2], chunk)
             if parts > 1:
                 scratch = torch.empty(n, dtype=torch.float32, device=q.device)
         _C().window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out, scale, H, window, pool, sink, v_freq, vt,
-                         prefill_kernel, bias_kind, bias_a, bias_b, gate, parts, scratch, softcap)
+                         prefill_kernel, bias_kind, bias_a, bias_b, gate, parts, scratch, softcap, chunk)
         return
     G, page, D, V = kc.shape[1], kc.shape[2], kc.shape[3], vc.shape[3]
     rep = H // G
@@ -602,7 +643,7 @@ def window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out,
         bt = block_tables[s]
         for t in range(t0, t1):
             i = pos0 + t - t0
-            lo = max(0, i - window + 1)
+            lo = max(0, i - window + 1, i - i % chunk if chunk else 0)
             pg, r = _seq_rows(bt, torch.arange(lo, i + 1), page)
             K, Vv = kc[pg, :, r].float(), vc[pg, :, r].float()           # [n, G, D], [n, value heads, V]
             if Vv.shape[1] != G:
