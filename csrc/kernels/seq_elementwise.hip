@@ -334,10 +334,10 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int32_t* __restric
 
 // x[t] += mult * u[t] (fp32 sum); with w: h[t] = norm(x[t]) * w from the new row. u[t]: the row of y, with GATHER the
 // weighted sum of the token's expert rows (choices ascending), with POST normed and weighted by post_w. CENTER: layer
-// norms. One workgroup per token; the row stays in registers between the norms and the add (W <= 256 * RN_MAX), the
-// columns beyond are read again.
-constexpr int RN_MAX = 16;
-template <bool POST, bool CENTER, bool GATHER>
+// norms. One workgroup per token; the first 256 NI columns stay in registers between the norms and the add, and what
+// does not depend on a norm (the stream's row, the weights) is asked for before the first of them; the columns beyond
+// are read again.
+template <int NI, bool POST, bool CENTER, bool GATHER>
 __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) {
   __shared__ float red[16];
   const int t = blockIdx.x, W = a.W, tid = threadIdx.x;
@@ -350,19 +350,48 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
       u = fmaf(a.wts[(int64_t)t * a.top + k], ldx(a.y, (int64_t)a.pos[(int64_t)t * a.top + k] * W + c, a.y_f32), u);
     return u;
   };
-  float keep[RN_MAX];
+  // every load of a register array is from a clamped column (never used past W), so none waits behind a branch
+  auto load_row = [&](int64_t ro, float (&u)[NI]) {
+    if (a.y_f32) {  // (uniform)
+#pragma unroll
+      for (int i = 0; i < NI; ++i) u[i] = reinterpret_cast<const float*>(a.y)[ro + min(tid + 256 * i, W - 1)];
+    } else {
+#pragma unroll
+      for (int i = 0; i < NI; ++i) u[i] = bf2f(reinterpret_cast<const bf16_t*>(a.y)[ro + min(tid + 256 * i, W - 1)]);
+    }
+  };
+  float keep[NI], xk[NI], pw[POST ? NI : 1], nw[NI];
+  if (GATHER) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) keep[i] = 0.f;
+    for (int k = 0; k < a.top; ++k) {  // a choice's loads for all columns of the thread are in flight together
+      const float wk = a.wts[(int64_t)t * a.top + k];
+      float u[NI];
+      load_row((int64_t)a.pos[(int64_t)t * a.top + k] * W, u);
+#pragma unroll
+      for (int i = 0; i < NI; ++i) keep[i] = fmaf(wk, u[i], keep[i]);
+    }
+  } else {
+    load_row((int64_t)t * W, keep);
+  }
+#pragma unroll
+  for (int i = 0; i < NI; ++i) xk[i] = xr[min(tid + 256 * i, W - 1)];
+  if (POST) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) pw[i] = a.post_w[min(tid + 256 * i, W - 1)];
+  }
+  if (a.w != nullptr) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) nw[i] = a.w[min(tid + 256 * i, W - 1)];
+  }
+  __syncthreads();  // (every thread has read its clamped columns before any of them is rewritten below)
   float pmean = 0.f, pinv = 1.f;
   if (POST) {
     float s = 0.f;
 #pragma unroll
-    for (int i = 0; i < RN_MAX; ++i) {
-      const int c = tid + 256 * i;
-      if (c < W) {
-        keep[i] = row(c);
-        s = CENTER ? s + keep[i] : fmaf(keep[i], keep[i], s);
-      }
-    }
-    for (int c = tid + 256 * RN_MAX; c < W; c += 256) {
+    for (int i = 0; i < NI; ++i)
+      if (tid + 256 * i < W) s = CENTER ? s + keep[i] : fmaf(keep[i], keep[i], s);
+    for (int c = tid + 256 * NI; c < W; c += 256) {
       const float u = row(c);
       s = CENTER ? s + u : fmaf(u, u, s);
     }
@@ -371,26 +400,26 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
       pmean = s / fw;
       s = 0.f;
 #pragma unroll
-      for (int i = 0; i < RN_MAX; ++i)
+      for (int i = 0; i < NI; ++i)
         if (tid + 256 * i < W) { const float d = keep[i] - pmean; s = fmaf(d, d, s); }
-      for (int c = tid + 256 * RN_MAX; c < W; c += 256) { const float d = row(c) - pmean; s = fmaf(d, d, s); }
+      for (int c = tid + 256 * NI; c < W; c += 256) { const float d = row(c) - pmean; s = fmaf(d, d, s); }
       s = block_reduce_sum(s, red);
     }
     pinv = 1.f / sqrtf(s / fw + a.eps);
   }
   float s = 0.f;
 #pragma unroll
-  for (int i = 0; i < RN_MAX; ++i) {
+  for (int i = 0; i < NI; ++i) {
     const int c = tid + 256 * i;
     if (c < W) {
-      const float u = POST ? (keep[i] - pmean) * pinv * a.post_w[c] : row(c);
-      const float v = fmaf(a.mult, u, xr[c]);
+      const float u = POST ? (keep[i] - pmean) * pinv * pw[POST ? i : 0] : keep[i];
+      const float v = fmaf(a.mult, u, xk[i]);
       xr[c] = v;
       keep[i] = v;
       s = CENTER ? s + v : fmaf(v, v, s);
     }
   }
-  for (int c = tid + 256 * RN_MAX; c < W; c += 256) {
+  for (int c = tid + 256 * NI; c < W; c += 256) {
     const float u = POST ? (row(c) - pmean) * pinv * a.post_w[c] : row(c);
     const float v = fmaf(a.mult, u, xr[c]);
     xr[c] = v;
@@ -403,18 +432,18 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
     mean = s / fw;
     s = 0.f;
 #pragma unroll
-    for (int i = 0; i < RN_MAX; ++i)
+    for (int i = 0; i < NI; ++i)
       if (tid + 256 * i < W) { const float d = keep[i] - mean; s = fmaf(d, d, s); }
-    for (int c = tid + 256 * RN_MAX; c < W; c += 256) { const float d = xr[c] - mean; s = fmaf(d, d, s); }
+    for (int c = tid + 256 * NI; c < W; c += 256) { const float d = xr[c] - mean; s = fmaf(d, d, s); }
     s = block_reduce_sum(s, red);
   }
   const float inv = 1.f / sqrtf(s / fw + a.eps);
 #pragma unroll
-  for (int i = 0; i < RN_MAX; ++i) {
+  for (int i = 0; i < NI; ++i) {
     const int c = tid + 256 * i;
-    if (c < W) stx(a.h, (int64_t)t * W + c, a.h_f32, (keep[i] - mean) * inv * a.w[c]);
+    if (c < W) stx(a.h, (int64_t)t * W + c, a.h_f32, (keep[i] - mean) * inv * nw[i]);
   }
-  for (int c = tid + 256 * RN_MAX; c < W; c += 256) stx(a.h, (int64_t)t * W + c, a.h_f32, (xr[c] - mean) * inv * a.w[c]);
+  for (int c = tid + 256 * NI; c < W; c += 256) stx(a.h, (int64_t)t * W + c, a.h_f32, (xr[c] - mean) * inv * a.w[c]);
 }
 
 // out[t] = [a[t], b[t]] in out's dtype
@@ -525,20 +554,26 @@ void launch_act_rows(const void* x, int64_t ldx_, void* out, int64_t ldo, int T,
                      reinterpret_cast<const bf16_t*>(x), ldx_, reinterpret_cast<bf16_t*>(out), ldo, n, act, total);
 }
 
-template <bool POST, bool CENTER>
+template <int NI, bool POST, bool CENTER>
 static void launch_residual_norm_as(const ResidualNormArgs& a, hipStream_t st) {
-  if (a.top > 0) hipLaunchKernelGGL((residual_norm_kernel<POST, CENTER, true>), dim3(a.T), dim3(256), 0, st, a);
-  else hipLaunchKernelGGL((residual_norm_kernel<POST, CENTER, false>), dim3(a.T), dim3(256), 0, st, a);
+  if (a.top > 0) hipLaunchKernelGGL((residual_norm_kernel<NI, POST, CENTER, true>), dim3(a.T), dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((residual_norm_kernel<NI, POST, CENTER, false>), dim3(a.T), dim3(256), 0, st, a);
+}
+template <int NI>
+static void launch_residual_norm_sized(const ResidualNormArgs& a, hipStream_t st) {
+  if (a.post_w != nullptr) {
+    if (a.center) launch_residual_norm_as<NI, true, true>(a, st);
+    else launch_residual_norm_as<NI, true, false>(a, st);
+  } else {
+    if (a.center) launch_residual_norm_as<NI, false, true>(a, st);
+    else launch_residual_norm_as<NI, false, false>(a, st);
+  }
 }
 void launch_residual_norm(const ResidualNormArgs& a, hipStream_t st) {
   if (a.T <= 0 || a.W <= 0) return;
-  if (a.post_w != nullptr) {
-    if (a.center) launch_residual_norm_as<true, true>(a, st);
-    else launch_residual_norm_as<true, false>(a, st);
-  } else {
-    if (a.center) launch_residual_norm_as<false, true>(a, st);
-    else launch_residual_norm_as<false, false>(a, st);
-  }
+  if (a.W <= 1024) launch_residual_norm_sized<4>(a, st);
+  else if (a.W <= 2048) launch_residual_norm_sized<8>(a, st);
+  else launch_residual_norm_sized<16>(a, st);
 }
 
 void launch_pair_rows(const float* a, const float* b, void* out, int out_f32, int T, int W, hipStream_t st) {

@@ -93,14 +93,14 @@ __global__ __launch_bounds__(256) void window_write_kernel(WindowArgs a, const v
   for (int e = tid; e < H * D; e += 256) xs[e] = ldx(q, (int64_t)t * ldq + e, a.f32);
   for (int e = tid; e < G * D; e += 256) xs[H * D + e] = ldx(k, (int64_t)t * ldk + e, a.f32);
   __syncthreads();
-  for (int h = wv; h < H + G; h += 4) {  // sum of squares per head
-    float ss = 0.f;
-    for (int d = lane; d < D; d += 64) ss = fmaf(xs[h * D + d], xs[h * D + d], ss);
-    ss = wave_reduce_sum(ss);
-    if (lane == 0) inv[h] = ss;
-  }
-  __syncthreads();
   if (qw != nullptr) {
+    for (int h = wv; h < H + G; h += 4) {  // sum of squares per head
+      float ss = 0.f;
+      for (int d = lane; d < D; d += 64) ss = fmaf(xs[h * D + d], xs[h * D + d], ss);
+      ss = wave_reduce_sum(ss);
+      if (lane == 0) inv[h] = ss;
+    }
+    __syncthreads();
     float mine = 0.f;
     if (norm_all) {
       float sq = 0.f, sk = 0.f;
