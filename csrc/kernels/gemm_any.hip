@@ -13,6 +13,7 @@
 //         32 staged through two LDS buffers, the next step's loads in flight during the current step's MFMAs.
 //   fp32: 64 x 64 x 16 LDS-tiled FMA kernel, 4 x 4 outputs per thread, k ascending.
 #include <cstdlib>
+#include <type_traits>
 
 #include "common.h"
 #include "seq_launchers.h"
@@ -42,18 +43,36 @@ __device__ __forceinline__ bool locate_tile(const AnyGemmArgs& p, int by, int& g
 
 __device__ __forceinline__ float sigmoidf_(float x) { return 1.f / (1.f + expf(-x)); }
 
-__device__ __forceinline__ float epi_val(const AnyGemmArgs& p, float g, float u) {
-  if (p.act == 1) return g * sigmoidf_(g) * u;
-  if (p.act == 2) {
+// the activation of one output (g: the accumulator with its bias, u: the second matrix's); ACT is AnyGemmArgs::act
+template <int ACT>
+__device__ __forceinline__ float act_val(const AnyGemmArgs& p, float g, float u) {
+  if (ACT == 1) return g * sigmoidf_(g) * u;
+  if (ACT == 2) {
     const float gg = fminf(g, p.limit);
     const float uu = fminf(fmaxf(u, -p.limit), p.limit);
     return gg * sigmoidf_(p.alpha * gg) * (uu + 1.f);
   }
-  if (p.act == 3) return tanhf(g);
-  if (p.act == 4) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
-  if (p.act == 5) return 0.5f * g * (1.f + erff(g * 0.70710678118654752f));
-  if (p.act == 6) { const float r = fmaxf(g, 0.f); return r * r; }
+  if (ACT == 3) return tanhf(g);
+  if (ACT == 4) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
+  if (ACT == 5) return 0.5f * g * (1.f + erff(g * 0.70710678118654752f));
+  if (ACT == 6) { const float r = fmaxf(g, 0.f); return r * r; }
   return g;
+}
+
+// fn<ACT>() for the launch's activation: one uniform branch per tile, so a thread's outputs run through straight code of
+// their own activation (a chain of tests per output would jump over every other activation's code each time)
+template <int DUAL, typename F>
+__device__ __forceinline__ void with_act(const AnyGemmArgs& p, F&& fn) {
+  if (DUAL) {
+    if (p.act == 1) fn(std::integral_constant<int, 1>{});
+    else if (p.act == 2) fn(std::integral_constant<int, 2>{});
+    else fn(std::integral_constant<int, 4>{});
+  } else {
+    if (p.act == 0) fn(std::integral_constant<int, 0>{});
+    else if (p.act == 6) fn(std::integral_constant<int, 6>{});
+    else if (p.act == 5) fn(std::integral_constant<int, 5>{});
+    else fn(std::integral_constant<int, 3>{});
+  }
 }
 
 __device__ __forceinline__ void store_out(const AnyGemmArgs& p, int64_t b, int m, int n, float v) {
@@ -213,20 +232,22 @@ __global__ __launch_bounds__(256) void gemm_any_mfma_kernel(AnyGemmArgs p) {
         if (DUAL) acc2[i][j] += red[KS ? wn : 0][KS ? 4 + 2 * i + j : 0][KS ? l : 0];
       }
   }
+  with_act<DUAL>(p, [&](auto act) {
 #pragma unroll
-  for (int i = 0; i < 2; ++i)
+    for (int i = 0; i < 2; ++i)
 #pragma unroll
-    for (int j = 0; j < NJ; ++j) {
-      const int n = n0 + wn * 16 * NJ + j * 16 + lr;
-      if (n >= p.N) continue;
-      const float bias = p.bias ? p.bias[n] : 0.f;
+      for (int j = 0; j < NJ; ++j) {
+        const int n = n0 + wn * 16 * NJ + j * 16 + lr;
+        if (n >= p.N) continue;
+        const float bias = p.bias ? p.bias[n] : 0.f;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int m = r0 + mrow + i * 16 + 4 * (l >> 4) + e;
-        if (m >= rend) continue;
-        store_out(p, b, m, n, epi_val(p, acc[i][j][e] + bias, DUAL ? acc2[i][j][e] : 0.f));
+        for (int e = 0; e < 4; ++e) {
+          const int m = r0 + mrow + i * 16 + 4 * (l >> 4) + e;
+          if (m >= rend) continue;
+          store_out(p, b, m, n, act_val<decltype(act)::value>(p, acc[i][j][e] + bias, DUAL ? acc2[i][j][e] : 0.f));
+        }
       }
-    }
+  });
 }
 
 // LDS-tiled form. Host-checked: K, the row strides and the batch strides are multiples of 8 elements, the bases
@@ -239,8 +260,12 @@ constexpr int LM = 128, LKS = 32, LPAD = LKS + 8;
 template <int DUAL>
 __global__ __launch_bounds__(256) void gemm_any_lds_kernel(AnyGemmArgs p) {
   constexpr int WN = DUAL ? 64 : 128;  // columns of each weight matrix per block
-  __shared__ __attribute__((aligned(16))) bf16_t As[2][LM][LPAD];
-  __shared__ __attribute__((aligned(16))) bf16_t Ws[2][128][LPAD];
+  constexpr int OPAD = WN + 8;         // padded row of the staged outputs
+  __shared__ __attribute__((aligned(16))) bf16_t smem[4 * LM * LPAD];  // two A and two weight buffers, then the outputs
+  static_assert(LM * OPAD <= 4 * LM * LPAD, "the staged outputs fit the operand buffers");
+  typedef bf16_t Tile[LM][LPAD];
+  Tile* As = reinterpret_cast<Tile*>(smem);
+  Tile* Ws = As + 2;
   int grp, r0, rend;
   if (!locate_tile(p, blockIdx.y, grp, r0, rend, LM)) return;
   const int64_t b = blockIdx.z;
@@ -310,20 +335,47 @@ __global__ __launch_bounds__(256) void gemm_any_lds_kernel(AnyGemmArgs p) {
     __syncthreads();
     buf ^= 1;
   }
+  if (p.vec_out) {  // bf16 rows of whole 16-B pieces: staged in LDS (the k loop's last barrier has freed it), then stored whole
+    with_act<DUAL>(p, [&](auto act) {
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+      for (int j = 0; j < (DUAL ? 2 : 4); ++j) {
+        const int col = (DUAL ? wn * 32 : wn * 64) + j * 16 + lr;
+        const float bias = p.bias ? p.bias[min(n0 + col, p.N - 1)] : 0.f;
 #pragma unroll
-    for (int j = 0; j < (DUAL ? 2 : 4); ++j) {
-      const int n = n0 + (DUAL ? wn * 32 : wn * 64) + j * 16 + lr;
-      if (n >= p.N) continue;
-      const float bias = p.bias ? p.bias[n] : 0.f;
+        for (int i = 0; i < 4; ++i)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int m = r0 + wm * 64 + i * 16 + 4 * lg + e;
-        if (m >= rend) continue;
-        store_out(p, b, m, n, epi_val(p, acc[i][j][e] + bias, DUAL ? acc[i][j + 2][e] : 0.f));
+          for (int e = 0; e < 4; ++e)
+            smem[(wm * 64 + i * 16 + 4 * lg + e) * OPAD + col] =
+                f2bf(act_val<decltype(act)::value>(p, acc[i][j][e] + bias, DUAL ? acc[i][j + 2][e] : 0.f));
       }
+    });
+    __syncthreads();
+    bf16_t* out = reinterpret_cast<bf16_t*>(p.out) + b * p.o_bs;
+#pragma unroll
+    for (int u = 0; u < LM * WN / 8 / 256; ++u) {
+      const int x = tid + 256 * u, row = x / (WN / 8), col = (x % (WN / 8)) * 8;
+      if (r0 + row < rend && n0 + col < p.N)
+        *reinterpret_cast<uint4*>(out + (int64_t)(r0 + row) * p.ldo + n0 + col) =
+            *reinterpret_cast<const uint4*>(&smem[row * OPAD + col]);
     }
+    return;
+  }
+  with_act<DUAL>(p, [&](auto act) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int j = 0; j < (DUAL ? 2 : 4); ++j) {
+        const int n = n0 + (DUAL ? wn * 32 : wn * 64) + j * 16 + lr;
+        if (n >= p.N) continue;
+        const float bias = p.bias ? p.bias[n] : 0.f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int m = r0 + wm * 64 + i * 16 + 4 * lg + e;
+          if (m >= rend) continue;
+          store_out(p, b, m, n, act_val<decltype(act)::value>(p, acc[i][j][e] + bias, DUAL ? acc[i][j + 2][e] : 0.f));
+        }
+      }
+  });
 }
 
 template <typename T>
@@ -394,18 +446,20 @@ __global__ __launch_bounds__(256) void gemm_any_fma_kernel(AnyGemmArgs p) {
     }
     __syncthreads();
   }
+  with_act<DUAL>(p, [&](auto act) {
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int m = r0 + ty * 4 + i;
-    if (m >= rend) continue;
+    for (int i = 0; i < 4; ++i) {
+      const int m = r0 + ty * 4 + i;
+      if (m >= rend) continue;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int n = n0 + tx * 4 + j;
-      if (n >= p.N) continue;
-      const float bias = p.bias ? p.bias[n] : 0.f;
-      store_out(p, b, m, n, epi_val(p, acc[i][j] + bias, DUAL ? acc2[i][j] : 0.f));
+      for (int j = 0; j < 4; ++j) {
+        const int n = n0 + tx * 4 + j;
+        if (n >= p.N) continue;
+        const float bias = p.bias ? p.bias[n] : 0.f;
+        store_out(p, b, m, n, act_val<decltype(act)::value>(p, acc[i][j] + bias, DUAL ? acc2[i][j] : 0.f));
+      }
     }
-  }
+  });
 }
 
 // "1": large products through the LDS-tiled kernel (default); "0": the direct-fragment kernels only
@@ -446,8 +500,10 @@ void launch_gemm_any(const AnyGemmArgs& g, hipStream_t st) {
     const dim3 gridw((g.N + 127) / 128, mt, g.batch);
     if (wide && g.M >= 1024 && lds_tiles()) {  // enough 128-row tiles
       const int mt128 = (g.M + LM - 1) / LM + (g.group_off ? g.groups : 0);
-      if (dual) hipLaunchKernelGGL((gemm_any_lds_kernel<1>), dim3((g.N + 63) / 64, mt128, g.batch), block, 0, st, g);
-      else hipLaunchKernelGGL((gemm_any_lds_kernel<0>), dim3((g.N + 127) / 128, mt128, g.batch), block, 0, st, g);
+      AnyGemmArgs v = g;
+      v.vec_out = !g.out_f32 && g.gate == nullptr && g.N % 8 == 0 && g.ldo % 8 == 0 && g.o_bs % 8 == 0 && a16(g.out);
+      if (dual) hipLaunchKernelGGL((gemm_any_lds_kernel<1>), dim3((g.N + 63) / 64, mt128, g.batch), block, 0, st, v);
+      else hipLaunchKernelGGL((gemm_any_lds_kernel<0>), dim3((g.N + 127) / 128, mt128, g.batch), block, 0, st, v);
     } else if (dual && wide) hipLaunchKernelGGL((gemm_any_mfma_kernel<1, true, 4>), gridw, block, 0, st, g);
     else if (wide) hipLaunchKernelGGL((gemm_any_mfma_kernel<0, true, 4>), gridw, block, 0, st, g);
     else if (dual && al) hipLaunchKernelGGL((gemm_any_mfma_kernel<1, true, 2>), grid, block, 0, st, g);

@@ -28,6 +28,7 @@ struct AnyGemmArgs {
                                         //   3 tanh, 5 gelu (erf form), 6 max(g, 0)^2
   float alpha = 1.702f;
   int in_f32 = 0, out_f32 = 0, gate_f32 = 0;
+  int vec_out = 0;                      // (set by launch_gemm_any: the outputs can be stored in 16-B pieces)
 };
 void launch_gemm_any(const AnyGemmArgs& g, hipStream_t st);
 
