@@ -449,7 +449,7 @@ def _chunk_reference(q, k, v, other, lam, gate, H, G, D, V, scale, dims, base, s
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("f32", [True, False])
 @pytest.mark.parametrize("H,G,D,V,dims,size", [(4, 2, 8, 16, 4, 37), (2, 2, 16, 8, 6, 16), (3, 1, 6, 5, 2, 100),
-                                               (2, 1, 160, 136, 32, 64), (2, 2, 96, 64, 24, 1000), (3, 3, 8, 8, 2, 1)])
+                                               (2, 1, 160, 136, 32, 64), (2, 2, 104, 72, 40, 1000), (3, 3, 8, 8, 2, 1)])
 def test_chunked_attention_on_crafted_keys(device, f32, H, G, D, V, dims, size):
     """The attention ops alone: for chosen query positions one key is made to dominate: the first key of the query's
     chunk, the last one before it (not seen), the token itself, keys at page borders, a key hundreds back. One
