@@ -77,7 +77,7 @@ __device__ __forceinline__ void with_act(const AnyGemmArgs& p, F&& fn) {
 
 __device__ __forceinline__ void store_out(const AnyGemmArgs& p, int64_t b, int m, int n, float v) {
   if (p.gate != nullptr) {
-    const int64_t gi = (int64_t)m * p.ldg + b * p.g_bs + n;
+    const int64_t gi = (int64_t)m * p.ldg + b * p.g_bs + (int64_t)n * p.g_cs;
     const float gl = p.gate_f32 ? reinterpret_cast<const float*>(p.gate)[gi]
                                 : bf2f(reinterpret_cast<const bf16_t*>(p.gate)[gi]);
     v *= sigmoidf_(gl);

@@ -6,8 +6,9 @@
 //   ol[t][h]       = sum_j softmax_j(score) c_j
 // A sink (one logit per head) only enters the softmax denominator: the running max starts at it, the sum at 1.
 // Key tiles sit at absolute positions whatever the window's start, so a row's sums keep their order.
-// latent_write: RMS norm of the latent (fp32 statistics) + interleaved-pair rotation of the shared key
-// part + the paged store, one launch. Angles are position * inv_freq in fp32 with full-range sin / cos.
+// latent_write: RMS norm of the latent (fp32 statistics) + rotation of the shared key part (interleaved or half-split
+// pairs, cos and sin times a factor) + the paged store, one launch. Angles are position * inv_freq in fp32 with
+// full-range sin / cos.
 // latent_attn, fp32 caches (and shapes the MFMA kernel does not take): one workgroup per (token, group
 // of heads); key tiles of 16 rows staged in LDS as fp32, scores, running max / sum and the weighted
 // latent sum all in fp32 FMA.
@@ -41,6 +42,18 @@ __device__ __forceinline__ void stx(void* p, int64_t i, int f32, float v) {
   else reinterpret_cast<bf16_t*>(p)[i] = f2bf(v);
 }
 
+// entry i (< rot_dims) of the row at x + base, turned by the position: pairs (2j, 2j + 1), or (j, j + rot_dims / 2)
+__device__ __forceinline__ float turned(const LatentArgs& a, const void* x, int64_t base, int i, float pos) {
+  const int hr = a.rot_dims >> 1;
+  const bool second = a.rot_half ? i >= hr : (i & 1);
+  const int j = a.rot_half ? (second ? i - hr : i) : (i >> 1);
+  const int i0 = a.rot_half ? j : (i & ~1), i1 = a.rot_half ? j + hr : (i | 1);
+  const float ang = pos * a.inv_freq[j];
+  const float cs = cosf(ang) * a.rot_amp, sn = sinf(ang) * a.rot_amp;
+  const float u = ldx(x, base + i0, a.f32), v = ldx(x, base + i1, a.f32);
+  return second ? (v * cs + u * sn) : (u * cs - v * sn);
+}
+
 __global__ __launch_bounds__(256) void latent_write_kernel(LatentArgs a, const void* __restrict__ kv, int64_t ldkv,
                                                             const float* __restrict__ w, float eps,
                                                             bf16_t* __restrict__ cache_t, int page) {
@@ -67,10 +80,7 @@ __global__ __launch_bounds__(256) void latent_write_kernel(LatentArgs a, const v
   for (int i = threadIdx.x; i < a.rot; i += blockDim.x) {
     float o;
     if (i < a.rot_dims) {
-      const float ang = pos * a.inv_freq[i >> 1];
-      const float cs = cosf(ang), sn = sinf(ang);
-      const float u = ldx(kv, src + a.rank + (i & ~1), a.f32), v = ldx(kv, src + a.rank + (i | 1), a.f32);
-      o = (i & 1) ? (v * cs + u * sn) : (u * cs - v * sn);
+      o = turned(a, kv, src + a.rank, i, pos);
     } else {
       o = ldx(kv, src + a.rank + i, a.f32);
     }
@@ -87,10 +97,7 @@ __global__ __launch_bounds__(256) void latent_qrope_kernel(LatentArgs a, const v
     const int64_t src = ((int64_t)t * H + h) * (dim + a.rot) + dim;
     float o;
     if (i < a.rot_dims) {
-      const float ang = pos * a.inv_freq[i >> 1];
-      const float cs = cosf(ang), sn = sinf(ang);
-      const float u = ldx(q, src + (i & ~1), a.f32), v = ldx(q, src + (i | 1), a.f32);
-      o = (i & 1) ? (v * cs + u * sn) : (u * cs - v * sn);
+      o = turned(a, q, src, i, pos);
     } else {
       o = ldx(q, src + i, a.f32);
     }

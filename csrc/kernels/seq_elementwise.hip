@@ -1,7 +1,8 @@
 // Row-wise kernels of layered hybrid models over an fp32 residual stream: embedding gather into
 // fp32, RMS or layer norm with a scalar or vector weight (fp32 statistics, bf16 or fp32 rows in and out,
 // optional row gather), a tanh norm without statistics, the gated residual update of a parallel layer,
-// the residual update of pre-norm and sandwich-norm layers with the next sublayer's norm,
+// the residual update of pre-norm and sandwich-norm layers with the next sublayer's norm, the one of layers whose
+// sublayers run side by side with both norms of the next layer,
 // the read / write of a sublayer over several learned-weight copies of the stream, and mixture-of-experts
 // routing (sigmoid or softmax scores with an optional selection-only correction, top-k, counting sort by
 // expert, weighted combine with an optional shared-expert row). Every kernel reads its sizes from arguments and its per-step metadata from device
@@ -446,6 +447,104 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
   for (int c = tid + 256 * NI; c < W; c += 256) stx(a.h, (int64_t)t * W + c, a.h_f32, (xr[c] - mean) * inv * a.w[c]);
 }
 
+// two sums over the workgroup at once (`red` needs 8 floats of LDS)
+__device__ __forceinline__ void block_sum2(float& a, float& b, float* red) {
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  a = wave_reduce_sum(a);
+  b = wave_reduce_sum(b);
+  __syncthreads();
+  if (lane == 0) { red[2 * wid] = a; red[2 * wid + 1] = b; }
+  __syncthreads();
+  a = red[0] + red[2] + red[4] + red[6];
+  b = red[1] + red[3] + red[5] + red[7];
+}
+
+// x[t] += s1 u1 + s2 u2 + y3 and the new row's norm under two weights. One workgroup per token; the first 256 NI columns
+// stay in registers between the norms, and every load that does not depend on a norm is asked for before the first of
+// them (from clamped columns, never used past W); the columns beyond are read again.
+template <int NI, bool BN>
+__global__ __launch_bounds__(256) void branch_residual_kernel(BranchResidualArgs a) {
+  __shared__ float red[16];
+  const int t = blockIdx.x, W = a.W, tid = threadIdx.x;
+  const int64_t ro = (int64_t)t * W;
+  float* xr = a.x + ro;
+  const float fw = (float)W;
+  float u1[NI], u2[NI], y[NI], w1[BN ? NI : 1], w2[BN ? NI : 1], n1[NI], n2[NI];
+  auto load = [&](const float* p, float (&v)[NI]) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) v[i] = p[min(tid + 256 * i, W - 1)];
+  };
+  auto load_or_zero = [&](const float* p, float (&v)[NI]) {
+    if (p != nullptr) load(p + ro, v);  // (uniform)
+    else {
+#pragma unroll
+      for (int i = 0; i < NI; ++i) v[i] = 0.f;
+    }
+  };
+  load_or_zero(a.y1, u1);
+  load_or_zero(a.y2, u2);
+  load_or_zero(a.y3, y);
+#pragma unroll
+  for (int i = 0; i < NI; ++i) y[i] += xr[min(tid + 256 * i, W - 1)];
+  if (BN) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      w1[BN ? i : 0] = a.w1[min(tid + 256 * i, W - 1)];
+      w2[BN ? i : 0] = a.w2[min(tid + 256 * i, W - 1)];
+    }
+  }
+  if (a.n1 != nullptr) load(a.n1, n1);
+  if (a.n2 != nullptr) load(a.n2, n2);
+  __syncthreads();  // (every thread has read its clamped columns before any of them is rewritten below)
+  float f1 = a.s1, f2 = a.s2;
+  if (BN) {
+    float q1 = 0.f, q2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < NI; ++i)
+      if (tid + 256 * i < W) { q1 = fmaf(u1[i], u1[i], q1); q2 = fmaf(u2[i], u2[i], q2); }
+    for (int c = tid + 256 * NI; c < W; c += 256) {
+      q1 = fmaf(a.y1[ro + c], a.y1[ro + c], q1);
+      q2 = fmaf(a.y2[ro + c], a.y2[ro + c], q2);
+    }
+    block_sum2(q1, q2, red);
+    f1 *= 1.f / sqrtf(q1 / fw + a.eps);
+    f2 *= 1.f / sqrtf(q2 / fw + a.eps);
+  }
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int c = tid + 256 * i;
+    if (c < W) {
+      const float v = y[i] + f1 * u1[i] * (BN ? w1[BN ? i : 0] : 1.f) + f2 * u2[i] * (BN ? w2[BN ? i : 0] : 1.f);
+      xr[c] = v;
+      y[i] = v;
+      s = fmaf(v, v, s);
+    }
+  }
+  for (int c = tid + 256 * NI; c < W; c += 256) {
+    float v = xr[c] + (a.y3 != nullptr ? a.y3[ro + c] : 0.f);
+    if (a.y1 != nullptr) v += f1 * a.y1[ro + c] * (BN ? a.w1[c] : 1.f);
+    if (a.y2 != nullptr) v += f2 * a.y2[ro + c] * (BN ? a.w2[c] : 1.f);
+    xr[c] = v;
+    s = fmaf(v, v, s);
+  }
+  if (a.n1 == nullptr) return;  // (uniform; n2 only beside n1)
+  s = block_reduce_sum(s, red);
+  const float inv = 1.f / sqrtf(s / fw + a.eps);
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int c = tid + 256 * i;
+    if (c < W) {
+      stx(a.h1, ro + c, a.h_f32, y[i] * inv * n1[i]);
+      if (a.n2 != nullptr) stx(a.h2, ro + c, a.h_f32, y[i] * inv * n2[i]);
+    }
+  }
+  for (int c = tid + 256 * NI; c < W; c += 256) {
+    stx(a.h1, ro + c, a.h_f32, xr[c] * inv * a.n1[c]);
+    if (a.n2 != nullptr) stx(a.h2, ro + c, a.h_f32, xr[c] * inv * a.n2[c]);
+  }
+}
+
 // out[t] = [a[t], b[t]] in out's dtype
 __global__ __launch_bounds__(256) void pair_rows_kernel(const float* __restrict__ a, const float* __restrict__ b,
                                                          void* __restrict__ out, int out_f32, int W, int64_t total) {
@@ -574,6 +673,18 @@ void launch_residual_norm(const ResidualNormArgs& a, hipStream_t st) {
   if (a.W <= 1024) launch_residual_norm_sized<4>(a, st);
   else if (a.W <= 2048) launch_residual_norm_sized<8>(a, st);
   else launch_residual_norm_sized<16>(a, st);
+}
+
+template <int NI>
+static void launch_branch_residual_sized(const BranchResidualArgs& a, hipStream_t st) {
+  if (a.w1 != nullptr) hipLaunchKernelGGL((branch_residual_kernel<NI, true>), dim3(a.T), dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((branch_residual_kernel<NI, false>), dim3(a.T), dim3(256), 0, st, a);
+}
+void launch_branch_residual(const BranchResidualArgs& a, hipStream_t st) {
+  if (a.T <= 0 || a.W <= 0) return;
+  if (a.W <= 1024) launch_branch_residual_sized<4>(a, st);
+  else if (a.W <= 2048) launch_branch_residual_sized<8>(a, st);
+  else launch_branch_residual_sized<16>(a, st);
 }
 
 void launch_pair_rows(const float* a, const float* b, void* out, int out_f32, int T, int W, hipStream_t st) {

@@ -19,6 +19,7 @@ struct AnyGemmArgs {
   int64_t ldw = 0, w_bs = 0;            // w_bs: stride between batches / groups
   const float* bias = nullptr;          // [N] added to the accumulator (single-matrix form)
   const void* gate = nullptr; int64_t ldg = 0, g_bs = 0;  // out *= sigmoid(gate[m][n]) (activation dtype)
+  int g_cs = 1;                         // the gate's column stride (0: one gate per row)
   void* out = nullptr; int64_t ldo = 0, o_bs = 0;
   int M = 0, N = 0, K = 0, batch = 1;
   const int32_t* group_off = nullptr;   // [groups + 1] row ranges (device): rows of group g use W + g * w_bs
@@ -65,6 +66,19 @@ struct ResidualNormArgs {
   int T = 0, W = 0;
 };
 void launch_residual_norm(const ResidualNormArgs& a, hipStream_t st);
+// x[t] += s1 u1[t] + s2 u2[t] + y3[t] in fp32 (any of y1, y2, y3 may be null), u_i = y_i, or with w1 (w2) given y_i divided
+// by sqrt(mean(y_i^2) + eps) times w_i [W]; then from the new row r = x[t] / sqrt(mean(x[t]^2) + eps):
+// h1[t] = r * n1 and h2[t] = r * n2 (each null: not made)
+struct BranchResidualArgs {
+  float* x = nullptr;
+  const float* y1 = nullptr; const float* y2 = nullptr; const float* y3 = nullptr;
+  float s1 = 1.f, s2 = 1.f, eps = 0.f;
+  const float* w1 = nullptr; const float* w2 = nullptr;
+  const float* n1 = nullptr; const float* n2 = nullptr;
+  void* h1 = nullptr; void* h2 = nullptr; int h_f32 = 0;
+  int T = 0, W = 0;
+};
+void launch_branch_residual(const BranchResidualArgs& a, hipStream_t st);
 // out[t] = [a[t], b[t]] (fp32 rows of W side by side) in out's dtype
 void launch_pair_rows(const float* a, const float* b, void* out, int out_f32, int T, int W, hipStream_t st);
 // out[k][t] = h[t] + (h'[t] - h[t]) * mu[k] for k < n blend vectors mu [n][W] (plane: stride between out's k planes),
@@ -94,6 +108,8 @@ void launch_post_norm_add(const PostNormArgs& a, hipStream_t st);
 
 struct LatentArgs {
   int rank = 0, rot = 0, rot_dims = 0;  // latent size, rotated key size, leading rotated dims (<= rot, even)
+  int rot_half = 0;                     // pairs (i, i + rot_dims / 2) instead of (2i, 2i + 1)
+  float rot_amp = 1.f;                  // factor on cos and sin
   const float* inv_freq = nullptr;      // [rot_dims / 2]
   const int32_t* positions = nullptr;   // [T]
   const int32_t* slots = nullptr;       // [T] cache row of each token (-1: padding)
@@ -142,6 +158,7 @@ struct WindowArgs {
   int page = 0, npool = 0;              // tokens per page; pooled rows per page (0: no pooled caches)
   int rot_dims = 0, window = 0, pool = 0;
   int chunk = 0;                        // c > 0: position i sees only j with floor(j / c) = floor(i / c) (not with pooled blocks)
+  int keep = 0;                         // the first `keep` positions are seen whatever the window (not with pooled blocks or chunks)
   int f32 = 0, T = 0, S = 0, max_blocks = 0;
   int prefill_kernel = 0;               // MFMA path, prompt portions: 0 LDS-staged tiles (64 rows), 1 split tiles (16 rows)
   const float* inv_freq = nullptr;      // [rot_dims / 2]
@@ -165,6 +182,7 @@ size_t window_attn_lds_bytes(const WindowArgs& a, int heads_per_block);
 // how many workgroups share a decoded token's key tiles (1: no split; only the bf16 MFMA kernel splits), and the
 // fp32 scratch elements window_attn then needs
 // (span: the most keys a position sees, 0 = not bounded)
+int window_attn_span(int window, int chunk, int keep, int pool);
 int window_attn_parts(int T, int S, int H, int G, int D, int V, int f32, int page, int span);
 int window_attn_nct(int D, int V);   // 16-column value tiles of the MFMA kernel instantiation for these head sizes
 size_t window_attn_part_floats(int T, int S, int H, int G, int D, int V, int parts);
@@ -216,6 +234,56 @@ int linear_attn_chunks(int T, int S, int CH);
 size_t linear_attn_scratch_floats(int T, int S, int H, int D, int V);
 // T rows; scratch: linear_attn_scratch_floats() floats, 16-B aligned
 void launch_linear_attn(const LinearAttnArgs& a, int T, float* scratch, hipStream_t st);
+
+// Gated delta rule over per-sequence state slots (gated_delta.hip).
+struct GatedDeltaArgs {
+  const void* q = nullptr; const void* k = nullptr; const void* v = nullptr; const void* b = nullptr;  // projections
+  int64_t ldq = 0, ldk = 0, ldv = 0, ldb = 0;   // activation dtype rows: q, k [G * D]; v [H * V]; b [H]
+  const float* z = nullptr; int64_t ldz = 0;    // [T][H * D] decay logits
+  const float* gate = nullptr; int64_t ldg = 0; // [T][H * V] output gate logits
+  const float* decay = nullptr;                 // [H]: g = exp(-decay softplus(z))
+  const float* nw = nullptr;                    // [V]
+  const float* conv_w = nullptr; int taps = 1;  // [taps][2 G D + H V]: q, k, v channels
+  float* conv_state = nullptr;                  // [slots][taps - 1][2 G D + H V]
+  float* state = nullptr;                       // [slots][H][D][V]
+  float unit_eps = 0.f, eps = 0.f, q_scale = 1.f;
+  const int32_t* state_slots = nullptr;         // [S] (-1: padding)
+  const int32_t* context_lens = nullptr; const int32_t* query_start = nullptr;
+  void* out = nullptr; int64_t ldo = 0;         // [T][H * V]
+  int S = 0, H = 0, G = 0, D = 0, V = 0, f32 = 0;
+  int wide = -1;                                // scan form: 1 several columns per lane, 0 one, -1 by the launch's size
+};
+size_t gated_delta_scratch_floats(int T, int H, int D, int V);
+void launch_gated_delta(const GatedDeltaArgs& a, int T, float* scratch, hipStream_t st);
+
+// Short causal convolution over time per channel and the selective scan behind it (selective_scan.hip).
+struct ShortConvArgs {
+  const void* x = nullptr; int64_t ldx = 0; int f32 = 0;   // [T][C] rows in the activation dtype
+  const float* w = nullptr; const float* b = nullptr;      // [taps][C] (last row: the current token), [C] or null
+  const float* kept = nullptr;                             // [slots][taps - 1][C] inputs before the step's portions
+  const int32_t* state_slots = nullptr; const int32_t* context_lens = nullptr; const int32_t* query_start = nullptr;
+  void* out = nullptr; int64_t ldo = 0;
+  int act = 0;                                             // 1: silu
+  int taps = 1, S = 0, T = 0, C = 0;
+};
+void launch_short_conv(const ShortConvArgs& a, hipStream_t st);
+struct SelectiveScanArgs {
+  const void* x = nullptr; int64_t ldx = 0;                // [T][C] convolved inputs
+  const float* dt = nullptr; int64_t lddt = 0;             // [T][C] steps before softplus
+  const void* B = nullptr; const void* Cm = nullptr; int64_t ldbc = 0;   // [T][N] each
+  const void* z = nullptr; int64_t ldz = 0;                // [T][C] gate
+  const float* A = nullptr;                                // [C][N]: A log2(e)
+  const float* D = nullptr;                                // [C]
+  float* state = nullptr;                                  // [slots][C][N]
+  const void* xin = nullptr; int64_t ldxin = 0;            // the convolution's inputs, for its kept rows
+  float* kept = nullptr; int taps = 1;                     // [slots][taps - 1][C]
+  const int32_t* state_slots = nullptr; const int32_t* context_lens = nullptr; const int32_t* query_start = nullptr;
+  void* out = nullptr; int64_t ldo = 0;
+  int S = 0, C = 0, N = 0, f32 = 0;
+};
+int selective_scan_chunk_size(int T, int S);
+size_t selective_scan_scratch_floats(int T, int S, int C, int N);
+void launch_selective_scan(const SelectiveScanArgs& a, int T, float* scratch, hipStream_t st);
 
 // idx, wts [T][top]: the `top` largest of s + corr with s by `score`: 0 sigmoid(z), 1 softmax(z) over all E;
 // wts = s of the chosen / (their sum + norm_eps) * scale. score 2: the `top` largest of z + corr, wts = softmax of z over

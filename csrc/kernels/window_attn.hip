@@ -40,6 +40,9 @@
 // Chunks (c > 0, not with pooled blocks): position i sees only the keys of its own chunk of c positions, counted from
 //               position 0 (first_key()); with a window too, the nearer of the two bounds holds. The key tiles a workgroup
 //               walks start at the chunk of its first row.
+// Kept first tokens (keep > 0, not with pooled blocks, chunks, a distance term or a softcap): the first `keep` positions
+//               are seen beside the window. Their key tiles (those before the window's first tile) come first (KEEP
+//               instantiations of the MFMA kernels); a tile that holds both kinds is one of the window's.
 // Value mixing: window_write can blend a token's values with another row of values of the same token (fp32).
 // Every row of every kernel depends only on its own sequence's cache rows, in an order fixed by the
 // position, so results do not depend on how a prompt is cut or what else is in the batch.
@@ -245,7 +248,10 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowArgs a, const vo
   const int tid = threadIdx.x;
   const int lo = max(0, first_key(a, pos));
   const int nb = a.pool > 0 ? max(0, pos - a.window + 1) / a.pool : 0;  // pooled blocks wholly before the window
-  const int nkeys = nb + (pos - lo + 1);
+  const int nf = min(a.keep, lo);                                       // kept first tokens before the window
+  const int nkeys = nb + nf + (pos - lo + 1);
+  // the token of key number e (counted after the pooled blocks): the kept first ones, then the window
+  auto token_of = [&](int e) { return e < nf ? e : lo + e - nf; };
   for (int e = tid; e < nh * D; e += 256) qs[(e / D) * DP + e % D] = ldx(q, ((int64_t)t * a.H + h0) * D + e, a.f32);
   if (tid < HC) {
     const bool sk = a.sink != nullptr && tid < nh;
@@ -271,7 +277,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowArgs a, const vo
           const int64_t row = ((int64_t)bt[e1 / page] * G + g) * a.npool + (e1 % page) / a.pool;
           val = ldx(isk ? a.kp : a.vp, row * w + ci, a.f32);
         } else {
-          const int j = lo + kj - nb;
+          const int j = token_of(kj - nb);
           const int64_t row = isk ? ((int64_t)bt[j / page] * G + g) * page + j % page
                                   : ((int64_t)bt[j / page] * a.GV + gv) * page + j % page;
           val = ldx(isk ? a.kc : a.vc, row * w + ci, a.f32);
@@ -294,7 +300,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowArgs a, const vo
       d += __shfl_xor(d, 1, 64);
       float bias = 0.f;
       if (a.bias_kind != 0 && on && j0 + jj >= nb && j0 + jj < nkeys) {  // (token keys: kj - nb keys after lo)
-        const int n = pos - (lo + j0 + jj - nb);
+        const int n = pos - token_of(j0 + jj - nb);
         bias = a.bias_kind == 1 ? -a.bias_a[h0 + h] * logf(1.f + a.bias_b[h0 + h] * (float)n)
                                 : a.bias_a[(int64_t)(h0 + h) * a.bias_n + min(n, a.bias_n - 1)];
       }
@@ -454,7 +460,7 @@ __device__ __forceinline__ float score_log2(const WindowArgs& a, float s, float 
   return a.cap_out * (1.f - 2.f / (e + 1.f));          // cap_out = cap log2e
 }
 
-template <int NCT, int NQF, int NW, int BIAS, bool CAP>
+template <int NCT, int NQF, int NW, int BIAS, bool CAP, bool KEEP>
 __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(WindowArgs a, const bf16_t* __restrict__ q,
                                                                 float scale_log2e, const bf16_t* __restrict__ vt,
                                                                 int num_pages, bf16_t* __restrict__ out) {
@@ -521,7 +527,8 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(WindowArgs a,
   const int klo = max(0, first_key(a, pmin));
   const int nbmax = P > 0 ? max(0, pmax - a.window + 1) / P : 0;
   const int ntp = (nbmax + 31) >> 5, jt0 = klo >> 5;
-  const int ntiles = ntp + (pmax >> 5) - jt0 + 1;
+  const int ntf = KEEP ? min((a.keep + 31) >> 5, jt0) : 0;  // tiles of kept first tokens before the window's tiles
+  const int ntiles = ntp + ntf + (pmax >> 5) - jt0 + 1;
   f32x4 O[NCT];
 #pragma unroll
   for (int ct = 0; ct < NCT; ++ct) O[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -541,7 +548,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(WindowArgs a,
       k0p = kp + (((int64_t)q0 * G + g) * a.npool + (e0 & 15) / P) * D;
       k1p = kp + (((int64_t)q1 * G + g) * a.npool + (e1 & 15) / P) * D;
     } else {
-      kbase = 32 * (jt0 + ti - ntp);
+      kbase = 32 * ((KEEP && ti - ntp < ntf) ? ti - ntp : jt0 + ti - ntp - ntf);
       pg0 = bt[kbase >> 4];
       pg1 = (kbase + 16 <= pmax) ? bt[(kbase >> 4) + 1] : pg0;
       pg0 = min(max(pg0, 0), num_pages - 1);
@@ -574,8 +581,8 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(WindowArgs a,
     if (BIAS) bias_tile(a, btab, g, rep, bw, bx, bo, bfar, hi, c0, kbase + 31 <= pmin - (a.bias_n - 1), bt0, bt1);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const bool vis0 = pooled ? c0 < nbv[i] : (c0 >= lo[i] && c0 <= hi[i]);
-      const bool vis1 = pooled ? c1 < nbv[i] : (c1 >= lo[i] && c1 <= hi[i]);
+      const bool vis0 = pooled ? c0 < nbv[i] : ((c0 >= lo[i] || (KEEP && c0 < a.keep)) && c0 <= hi[i]);
+      const bool vis1 = pooled ? c1 < nbv[i] : ((c1 >= lo[i] || (KEEP && c1 < a.keep)) && c1 <= hi[i]);
       const float v0 = vis0 ? score_log2<CAP>(a, s0[i], scale_log2e, BIAS ? bt0[i] : 0.f) : -INFINITY;
       const float v1 = vis1 ? score_log2<CAP>(a, s1[i], scale_log2e, BIAS ? bt1[i] : 0.f) : -INFINITY;
       const float mnew = fmaxf(m[i], group16_max(fmaxf(v0, v1)));
@@ -770,7 +777,7 @@ __global__ __launch_bounds__(256) void window_attn_merge_kernel(WindowArgs a, in
 // and transposed values are brought into LDS once per workgroup (two buffers: tile t + 1 is asked for before
 // tile t is computed, written after it, one barrier per tile), and every wave takes its fragments from there.
 // Pooled tiles come first and are read straight from the pooled caches by each wave, as in the kernel above.
-template <int NCT, int NQF, int BIAS, bool CAP>
+template <int NCT, int NQF, int BIAS, bool CAP, bool KEEP>
 __global__ __launch_bounds__(256) void window_attn_tiled_kernel(WindowArgs a, const bf16_t* __restrict__ q,
                                                                  float scale_log2e, const bf16_t* __restrict__ vt,
                                                                  int num_pages, bf16_t* __restrict__ out) {
@@ -858,8 +865,8 @@ __global__ __launch_bounds__(256) void window_attn_tiled_kernel(WindowArgs a, co
     if (BIAS) bias_tile(a, btab, g, rep, bw, bx, bo, bfar, hi, c0, kbase + 31 <= pminw - (a.bias_n - 1), bt0, bt1);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const bool vis0 = pooled ? c0 < nbv[i] : (c0 >= lo[i] && c0 <= hi[i]);
-      const bool vis1 = pooled ? c1 < nbv[i] : (c1 >= lo[i] && c1 <= hi[i]);
+      const bool vis0 = pooled ? c0 < nbv[i] : ((c0 >= lo[i] || (KEEP && c0 < a.keep)) && c0 <= hi[i]);
+      const bool vis1 = pooled ? c1 < nbv[i] : ((c1 >= lo[i] || (KEEP && c1 < a.keep)) && c1 <= hi[i]);
       const float v0 = vis0 ? score_log2<CAP>(a, s0[i], scale_log2e, BIAS ? bt0[i] : 0.f) : -INFINITY;
       const float v1 = vis1 ? score_log2<CAP>(a, s1[i], scale_log2e, BIAS ? bt1[i] : 0.f) : -INFINITY;
       const float mnew = fmaxf(m[i], group16_max(fmaxf(v0, v1)));
@@ -952,16 +959,19 @@ __global__ __launch_bounds__(256) void window_attn_tiled_kernel(WindowArgs a, co
     }
   };
   __syncthreads();  // the zero fill is done before the first tile is staged
-  fetch(jt0);
+  const int ntf = KEEP ? min((a.keep + 31) >> 5, jt0) : 0;  // tiles of kept first tokens, then the window's
+  const int ntiles = ntf + jt1 - jt0 + 1;
+  auto tile_of = [&](int it) { return (KEEP && it < ntf) ? it : jt0 + it - ntf; };
+  fetch(tile_of(0));
   int buf = 0;
   // a buffer is rewritten two tiles later, after the barrier of the tile in between, which every wave
   // reaches only when it has finished reading it
-  for (int jt = jt0; jt <= jt1; ++jt) {
+  for (int it = 0; it < ntiles; ++it) {
     stage(buf);
     __syncthreads();
-    if (jt < jt1) fetch(jt + 1);
-    const int kbase = 32 * jt;
-    if (active && kbase + 31 >= klow && kbase <= pmaxw) {  // wave-uniform: some row of the wave may see the tile
+    if (it + 1 < ntiles) fetch(tile_of(it + 1));
+    const int kbase = 32 * tile_of(it);
+    if (active && (kbase + 31 >= klow || (KEEP && kbase < a.keep)) && kbase <= pmaxw) {  // wave-uniform: some row of the wave may see the tile
       f32x4 s0 = f32x4{0.f, 0.f, 0.f, 0.f}, s1 = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kk = 0; kk < NQF; ++kk)
@@ -1007,7 +1017,7 @@ __global__ __launch_bounds__(256) void window_attn_tiled_kernel(WindowArgs a, co
   }
 }
 
-template <int NCT, int NQF, int BIAS, bool CAP>
+template <int NCT, int NQF, int BIAS, bool CAP, bool KEEP>
 void launch_window_mfma(const WindowArgs& a, const void* q, float scale, const void* vt, int num_pages, void* out,
                         hipStream_t st) {
   const int rep = a.H / a.G;
@@ -1022,14 +1032,14 @@ void launch_window_mfma(const WindowArgs& a, const void* q, float scale, const v
   // 16 rows per workgroup with the key tiles shared out over four waves)
   if ((int64_t)a.T * rep <= 16 * (int64_t)a.S) {
     const int parts = a.parts > 1 ? a.parts : 1;
-    hipLaunchKernelGGL((window_attn_mfma_kernel<NCT, NQF, 8, BIAS, CAP>), dim3(blocks, a.G, parts), dim3(512), dyn, st, a, qp, sl, vp,
+    hipLaunchKernelGGL((window_attn_mfma_kernel<NCT, NQF, 8, BIAS, CAP, KEEP>), dim3(blocks, a.G, parts), dim3(512), dyn, st, a, qp, sl, vp,
                        num_pages, op);
     if (parts > 1) hipLaunchKernelGGL(window_attn_merge_kernel, dim3(blocks, a.G, 4), dim3(256), 0, st, a, 16 * NCT, op);
   }
   else if (a.prefill_kernel == 1 || NCT > 8)
-    hipLaunchKernelGGL((window_attn_mfma_kernel<NCT, NQF, 4, BIAS, CAP>), dim3(blocks, a.G), dim3(256), dyn, st, a, qp, sl, vp, num_pages, op);
+    hipLaunchKernelGGL((window_attn_mfma_kernel<NCT, NQF, 4, BIAS, CAP, KEEP>), dim3(blocks, a.G), dim3(256), dyn, st, a, qp, sl, vp, num_pages, op);
   else
-    hipLaunchKernelGGL((window_attn_tiled_kernel<NCT, NQF, BIAS, CAP>), dim3((a.T * rep + 63) / 64 + a.S, a.G), dim3(256), dyn, st, a, qp, sl,
+    hipLaunchKernelGGL((window_attn_tiled_kernel<NCT, NQF, BIAS, CAP, KEEP>), dim3((a.T * rep + 63) / 64 + a.S, a.G), dim3(256), dyn, st, a, qp, sl,
                        vp, num_pages, op);
 }
 
@@ -1037,13 +1047,13 @@ void launch_window_mfma(const WindowArgs& a, const void* q, float scale, const v
 int window_attn_nct(int D, int V);
 namespace {
 
-template <int BIAS, bool CAP>
+template <int BIAS, bool CAP, bool KEEP>
 void launch_window_mfma_sized(const WindowArgs& a, const void* q, float scale, const void* vt, int num_pages, void* out,
                               hipStream_t st) {
   const int nct = window_attn_nct(a.D, a.V);  // (the scratch of a split launch is sized by the same rule)
-  if (nct == 4) launch_window_mfma<4, 2, BIAS, CAP>(a, q, scale, vt, num_pages, out, st);
-  else if (nct == 8) launch_window_mfma<8, 4, BIAS, CAP>(a, q, scale, vt, num_pages, out, st);
-  else launch_window_mfma<16, 8, BIAS, CAP>(a, q, scale, vt, num_pages, out, st);
+  if (nct == 4) launch_window_mfma<4, 2, BIAS, CAP, KEEP>(a, q, scale, vt, num_pages, out, st);
+  else if (nct == 8) launch_window_mfma<8, 4, BIAS, CAP, KEEP>(a, q, scale, vt, num_pages, out, st);
+  else launch_window_mfma<16, 8, BIAS, CAP, KEEP>(a, q, scale, vt, num_pages, out, st);
 }
 
 int heads_per_block(const WindowArgs& a) {
@@ -1066,6 +1076,11 @@ int window_attn_parts(int T, int S, int H, int G, int D, int V, int f32, int pag
   int parts = 512 / (wg > 0 ? wg : 1);
   if (span > 0) parts = std::min(parts, (span / 32 + 1 + 7) / 8);
   return parts < 2 ? 1 : (parts > 8 ? 8 : parts);
+}
+// the most keys a position sees (0: not bounded): tiles of a window can start and end anywhere, and so can the kept ones
+int window_attn_span(int window, int chunk, int keep, int pool) {
+  if (chunk > 0) return chunk;
+  return (pool == 0 && window < (1 << 20) && keep < (1 << 20)) ? window + (keep > 0 ? keep + 32 : 0) : 0;
 }
 int window_attn_nct(int D, int V) { return (D <= 64 && V <= 64) ? 4 : ((D <= 128 && V <= 128) ? 8 : 16); }
 size_t window_attn_part_floats(int T, int S, int H, int G, int D, int V, int parts) {
@@ -1107,9 +1122,10 @@ void launch_window_attn(const WindowArgs& a0, const void* q, float scale, void* 
   WindowArgs a = a0;
   if (a.softcap > 0.f) { a.cap_in = 2.f / a.softcap; a.cap_out = a.softcap * 1.4426950408889634f; }
   if (!a.f32 && vt != nullptr && a.page == 16 && a.D % 8 == 0 && a.D >= 8 && a.D <= 256 && a.V <= 256) {
-    if (a.bias_kind != 0) launch_window_mfma_sized<1, false>(a, q, scale, vt, num_pages, out, st);
-    else if (a.softcap > 0.f) launch_window_mfma_sized<0, true>(a, q, scale, vt, num_pages, out, st);
-    else launch_window_mfma_sized<0, false>(a, q, scale, vt, num_pages, out, st);
+    if (a.keep > 0) launch_window_mfma_sized<0, false, true>(a, q, scale, vt, num_pages, out, st);  // (host-checked: no term, no softcap)
+    else if (a.bias_kind != 0) launch_window_mfma_sized<1, false, false>(a, q, scale, vt, num_pages, out, st);
+    else if (a.softcap > 0.f) launch_window_mfma_sized<0, true, false>(a, q, scale, vt, num_pages, out, st);
+    else launch_window_mfma_sized<0, false, false>(a, q, scale, vt, num_pages, out, st);
     return;
   }
   const int HC = heads_per_block(a);

@@ -73,8 +73,12 @@ void gemm_any(const Tensor& a, const Tensor& w, Tensor& out, const OptT& w2, con
   g.bias = f32p(bias, "bias", g.N);
   TORCH_CHECK(!(g.bias && B > 1), "gemm_any: bias only without batch");
   if (has(gate)) {
-    g.gate_f32 = act_f32(*gate, "gate");
+    TORCH_CHECK(gate->is_cuda() && (gate->scalar_type() == torch::kFloat32 || gate->scalar_type() == torch::kBFloat16),
+                "gemm_any: gate bf16 or fp32 on the GPU");
+    g.gate_f32 = gate->scalar_type() == torch::kFloat32 ? 1 : 0;
     TORCH_CHECK(gate->dim() == out.dim() && gate->size(-1) == g.N && gate->size(-2) >= g.M, "gemm_any: gate shape");
+    TORCH_CHECK(gate->stride(-1) == 1 || gate->stride(-1) == 0 || g.N == 1, "gemm_any: gate columns adjacent, or one per row (expanded)");
+    g.g_cs = (int)gate->stride(-1);
     g.gate = gate->data_ptr(); g.ldg = gate->stride(-2); g.g_bs = b3 ? gate->stride(0) : 0;
   }
   const int64_t rows_in = a.size(-2);
@@ -143,8 +147,9 @@ void gated_residual(Tensor& x, const Tensor& y1, const OptT& g1, const OptT& b1,
 }
 
 vgate::LatentArgs latent_common(const Tensor& positions, const Tensor& inv_freq, int64_t rot_dims, int64_t rank,
-                                int64_t rot, int64_t T) {
+                                int64_t rot, int64_t T, bool rot_half, double rot_amp) {
   vgate::LatentArgs a;
+  a.rot_half = rot_half ? 1 : 0; a.rot_amp = (float)rot_amp;
   a.rank = (int)rank; a.rot = (int)rot; a.rot_dims = (int)rot_dims; a.T = (int)T;
   TORCH_CHECK(rank > 0 && rot >= 0 && rot_dims >= 0 && rot_dims <= rot && rot_dims % 2 == 0, "latent: rank / rot sizes");
   OptT f(inv_freq);
@@ -154,13 +159,14 @@ vgate::LatentArgs latent_common(const Tensor& positions, const Tensor& inv_freq,
 }
 
 void latent_write(const Tensor& kv, const Tensor& w, double eps, const Tensor& positions, const Tensor& slots,
-                  const Tensor& inv_freq, int64_t rot_dims, Tensor& cache, int64_t rank, const OptT& cache_t) {
+                  const Tensor& inv_freq, int64_t rot_dims, Tensor& cache, int64_t rank, const OptT& cache_t, bool rot_half,
+                  double rot_amp) {
   const int f = act_f32(kv, "kv");
   TORCH_CHECK(kv.dim() == 2 && cache.dim() == 3 && cache.is_contiguous() && act_f32(cache, "cache") == f,
               "latent_write: kv [T, rank + rot], cache [pages, page, rank + rot] of one dtype");
   const int64_t rot = kv.size(1) - rank;
   TORCH_CHECK(cache.size(2) == kv.size(1), "latent_write: cache row width");
-  auto a = latent_common(positions, inv_freq, rot_dims, rank, rot, kv.size(0));
+  auto a = latent_common(positions, inv_freq, rot_dims, rank, rot, kv.size(0), rot_half, rot_amp);
   a.slots = i32p(slots, "slots", kv.size(0));  // values < pages * page: written by the step's block tables
   a.cache = cache.data_ptr(); a.f32 = f;
   OptT wo(w);
@@ -176,12 +182,12 @@ void latent_write(const Tensor& kv, const Tensor& w, double eps, const Tensor& p
 }
 
 void latent_qrope(const Tensor& q, const Tensor& positions, const Tensor& inv_freq, int64_t rot_dims, Tensor& qa,
-                  int64_t H, int64_t dim, int64_t rank, int64_t rot) {
+                  int64_t H, int64_t dim, int64_t rank, int64_t rot, bool rot_half, double rot_amp) {
   const int f = act_f32(q, "q");
   TORCH_CHECK(q.dim() == 2 && q.is_contiguous() && q.size(1) == H * (dim + rot), "latent_qrope: q [T, H * (dim + rot)]");
   TORCH_CHECK(act_f32(qa, "qa") == f && qa.is_contiguous() && qa.numel() == q.size(0) * H * (rank + rot),
               "latent_qrope: qa [T, H, rank + rot]");
-  auto a = latent_common(positions, inv_freq, rot_dims, rank, rot, q.size(0));
+  auto a = latent_common(positions, inv_freq, rot_dims, rank, rot, q.size(0), rot_half, rot_amp);
   a.f32 = f;
   c10::DeviceGuard guard(q.device());
   vgate::launch_latent_qrope(a, q.data_ptr(), (int)H, (int)dim, qa.data_ptr(), cur_stream());
@@ -330,6 +336,38 @@ void residual_norm(Tensor& x, const Tensor& y, double mult, const OptT& w, doubl
   a.T = (int)T; a.W = (int)W;
   c10::DeviceGuard guard(x.device());
   vgate::launch_residual_norm(a, cur_stream());
+}
+
+// y1 .. y3 fp32 [T, W]; w1, w2: norms of y1 / y2 (both or neither); n1 / h1 and n2 / h2: the new row's norm, twice
+void branch_residual(Tensor& x, const OptT& y1, double s1, const OptT& w1, const OptT& y2, double s2, const OptT& w2,
+                     const OptT& y3, double eps, const OptT& n1, const OptT& h1, const OptT& n2, const OptT& h2, int64_t T) {
+  TORCH_CHECK(x.is_cuda() && x.scalar_type() == torch::kFloat32 && x.is_contiguous() && x.dim() == 2 && T >= 0 && T <= x.size(0),
+              "branch_residual: x fp32 [>= T, W]");
+  vgate::BranchResidualArgs a;
+  const int64_t W = x.size(1);
+  auto row = [&](const OptT& y, const char* name) -> const float* {
+    if (!has(y)) return nullptr;
+    TORCH_CHECK(y->is_cuda() && y->scalar_type() == torch::kFloat32 && y->is_contiguous() && y->dim() == 2 && y->size(0) >= T &&
+                y->size(1) == W, "branch_residual: ", name, " fp32 [>= T, W]");
+    return y->data_ptr<float>();
+  };
+  a.x = x.data_ptr<float>();
+  a.y1 = row(y1, "y1"); a.y2 = row(y2, "y2"); a.y3 = row(y3, "y3");
+  TORCH_CHECK(has(w1) == has(w2) && (!has(w1) || (has(y1) && has(y2))), "branch_residual: both branches are normed or neither");
+  a.w1 = f32p(w1, "w1", W); a.w2 = f32p(w2, "w2", W);
+  a.s1 = (float)s1; a.s2 = (float)s2; a.eps = (float)eps;
+  TORCH_CHECK(has(n1) == has(h1) && has(n2) == has(h2) && (!has(n2) || has(n1)), "branch_residual: a norm weight and its output come together");
+  a.n1 = f32p(n1, "n1", W); a.n2 = f32p(n2, "n2", W);
+  for (const OptT* h : {&h1, &h2}) {
+    if (!has(*h)) continue;
+    const int f = act_f32(**h, "h");
+    TORCH_CHECK((*h)->dim() == 2 && (*h)->is_contiguous() && (*h)->size(1) == W && (*h)->size(0) >= T, "branch_residual: h [>= T, W]");
+    if (h == &h1) { a.h1 = (*h)->data_ptr(); a.h_f32 = f; }
+    else { a.h2 = (*h)->data_ptr(); TORCH_CHECK(f == a.h_f32, "branch_residual: h1 and h2 of one dtype"); }
+  }
+  a.T = (int)T; a.W = (int)W;
+  c10::DeviceGuard guard(x.device());
+  vgate::launch_branch_residual(a, cur_stream());
 }
 
 void pair_rows(const Tensor& a, const Tensor& b, Tensor& out) {
@@ -522,10 +560,13 @@ void window_attn(const Tensor& q, const Tensor& kc, const Tensor& vc, const OptT
                  const Tensor& block_tables, const Tensor& context_lens, const Tensor& query_start, Tensor& out,
                  double scale, int64_t H, int64_t window, int64_t pool, const OptT& sink, const OptT& v_freq, const OptT& vt,
                  int64_t prefill_kernel, int64_t bias_kind, const OptT& bias_a, const OptT& bias_b, const OptT& gate,
-                 int64_t parts, const OptT& part_scratch, double softcap, int64_t chunk) {
+                 int64_t parts, const OptT& part_scratch, double softcap, int64_t chunk, int64_t keep) {
   auto a = window_common(kc, vc, kp, vp, H, pool);
   TORCH_CHECK(chunk >= 0 && chunk <= (1 << 30) && (chunk == 0 || pool == 0), "window_attn: chunk 0 (none) .. 2^30, not with pooled blocks");
   a.chunk = (int)chunk;
+  TORCH_CHECK(keep >= 0 && keep <= (1 << 30) && (keep == 0 || (pool == 0 && chunk == 0 && bias_kind == 0 && softcap == 0.0)),
+              "window_attn: keep 0 (none) .. 2^30, not with pooled blocks, chunks, a distance term or a softcap");
+  a.keep = (int)keep;
   TORCH_CHECK(softcap >= 0.0 && (softcap == 0.0 || bias_kind == 0), "window_attn: softcap >= 0, not with a distance term");
   a.softcap = (float)softcap;
   window_seq_meta(a, block_tables, query_start);
@@ -562,7 +603,8 @@ void window_attn(const Tensor& q, const Tensor& kc, const Tensor& vc, const OptT
   a.v_freq = f32p(v_freq, "v_freq", a.V / 2);
   const void* vtp = window_vt(vt, vc);
   if (parts > 1) {  // only what window_attn_parts() allows for this launch, with its scratch
-    TORCH_CHECK(vtp != nullptr && parts == vgate::window_attn_parts((int)T, a.S, a.H, a.G, a.D, a.V, a.f32, a.page, a.chunk),
+    TORCH_CHECK(vtp != nullptr && parts == vgate::window_attn_parts((int)T, a.S, a.H, a.G, a.D, a.V, a.f32, a.page,
+                                                                     vgate::window_attn_span(a.window, a.chunk, a.keep, a.pool)),
                 "window_attn: parts must be window_attn_split()'s for this step");
     const size_t need = vgate::window_attn_part_floats((int)T, a.S, a.H, a.G, a.D, a.V, (int)parts);
     TORCH_CHECK(has(part_scratch) && part_scratch->is_cuda() && part_scratch->scalar_type() == torch::kFloat32 &&
@@ -635,6 +677,127 @@ void linear_attn(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor
   TORCH_CHECK((reinterpret_cast<uintptr_t>(scratch.data_ptr()) & 15) == 0, "linear_attn: scratch must be 16-B aligned");
   c10::DeviceGuard guard(q.device());
   vgate::launch_linear_attn(p, (int)T, scratch.data_ptr<float>(), cur_stream());
+}
+
+const int32_t* slots_of(const Tensor& state_slots, int S) { return i32p(state_slots, "state_slots", S); }  // values < slots, or -1
+
+// q, k [T, G D], v [T, H V], b [T, H] column views of the step's projection; z fp32 [T, H D], gate fp32 [T, H V]
+void gated_delta(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& b, const Tensor& z, const Tensor& gate,
+                 const Tensor& decay, const Tensor& nw, const Tensor& conv_w, Tensor& state, Tensor& conv_state,
+                 const Tensor& state_slots, const Tensor& context_lens, const Tensor& query_start, Tensor& out, double unit_eps,
+                 double q_scale, double eps, Tensor& scratch, int64_t wide) {
+  vgate::GatedDeltaArgs p;
+  p.f32 = act_f32(q, "q");
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == torch::kFloat32 && state.is_contiguous() && state.dim() == 4,
+              "gated_delta: state fp32 [slots, H, D, V]");
+  p.H = (int)state.size(1); p.D = (int)state.size(2); p.V = (int)state.size(3);
+  const int64_t T = q.size(0), HD = (int64_t)p.H * p.D, HV = (int64_t)p.H * p.V;
+  TORCH_CHECK(p.D >= 1 && p.D <= 256 && p.V >= 1, "gated_delta: key size 1..256");
+  TORCH_CHECK(q.dim() == 2 && q.size(1) % p.D == 0 && q.size(1) >= p.D, "gated_delta: q [T, G * D]");
+  p.G = (int)(q.size(1) / p.D);
+  TORCH_CHECK(p.H % p.G == 0 && p.G <= 65535 && p.H <= 65535, "gated_delta: heads a multiple of query / key heads");
+  auto rows = [&](const Tensor& t, int64_t n, const char* name) {
+    TORCH_CHECK(act_f32(t, name) == p.f32 && t.dim() == 2 && t.size(0) == T && t.size(1) == n, "gated_delta: ", name, " [T, ", n, "]");
+  };
+  rows(q, (int64_t)p.G * p.D, "q"); rows(k, (int64_t)p.G * p.D, "k"); rows(v, HV, "v"); rows(b, p.H, "b"); rows(out, HV, "out");
+  p.q = q.data_ptr(); p.k = k.data_ptr(); p.v = v.data_ptr(); p.b = b.data_ptr();
+  p.ldq = q.stride(0); p.ldk = k.stride(0); p.ldv = v.stride(0); p.ldb = b.stride(0);
+  p.out = out.data_ptr(); p.ldo = out.stride(0);
+  auto logits = [&](const Tensor& t, int64_t n, const char* name) {
+    TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kFloat32 && t.dim() == 2 && t.stride(1) == 1 && t.size(0) == T &&
+                t.size(1) == n, "gated_delta: ", name, " fp32 [T, ", n, "]");
+  };
+  logits(z, HD, "z"); logits(gate, HV, "gate");
+  p.z = z.data_ptr<float>(); p.ldz = z.stride(0); p.gate = gate.data_ptr<float>(); p.ldg = gate.stride(0);
+  const int64_t NC = 2 * (int64_t)p.G * p.D + HV;
+  TORCH_CHECK(conv_w.dim() == 2 && conv_w.size(1) == NC && conv_w.size(0) >= 1 && conv_w.size(0) <= 4096,
+              "gated_delta: conv_w [taps, 2 G D + H V]");
+  p.taps = (int)conv_w.size(0);
+  OptT o0(decay), o1(nw), o2(conv_w);
+  p.decay = f32p(o0, "decay", p.H); p.nw = f32p(o1, "nw", p.V); p.conv_w = f32p(o2, "conv_w", p.taps * NC);
+  TORCH_CHECK(conv_state.is_cuda() && conv_state.scalar_type() == torch::kFloat32 && conv_state.is_contiguous() &&
+              conv_state.dim() == 3 && conv_state.size(0) == state.size(0) && conv_state.size(1) == p.taps - 1 &&
+              conv_state.size(2) == NC, "gated_delta: conv_state fp32 [slots, taps - 1, 2 G D + H V]");
+  p.conv_state = p.taps > 1 ? conv_state.data_ptr<float>() : nullptr;
+  p.state = state.data_ptr<float>();
+  p.unit_eps = (float)unit_eps; p.q_scale = (float)q_scale; p.eps = (float)eps;
+  p.S = (int)state_slots.numel();
+  p.state_slots = slots_of(state_slots, p.S);
+  p.context_lens = i32p(context_lens, "context_lens", p.S);
+  p.query_start = i32p(query_start, "query_start", p.S + 1);  // values <= T: set by the step metadata
+  TORCH_CHECK(scratch.is_cuda() && scratch.scalar_type() == torch::kFloat32 && scratch.is_contiguous() &&
+              (size_t)scratch.numel() >= vgate::gated_delta_scratch_floats((int)T, p.H, p.D, p.V) &&
+              (reinterpret_cast<uintptr_t>(scratch.data_ptr()) & 15) == 0,
+              "gated_delta: scratch fp32 with T * H * (4 D + 2 V) elements, 16-B aligned");
+  p.wide = (int)wide;
+  c10::DeviceGuard guard(q.device());
+  vgate::launch_gated_delta(p, (int)T, scratch.data_ptr<float>(), cur_stream());
+}
+
+const float* kept_rows(const Tensor& kept, int64_t taps, int64_t C) {
+  TORCH_CHECK(kept.is_cuda() && kept.scalar_type() == torch::kFloat32 && kept.is_contiguous() && kept.dim() == 3 &&
+              kept.size(1) == taps - 1 && kept.size(2) == C, "kept convolution inputs: fp32 [slots, taps - 1, C]");
+  return taps > 1 ? kept.data_ptr<float>() : nullptr;
+}
+
+void short_conv(const Tensor& x, const Tensor& w, const OptT& b, const Tensor& kept, const Tensor& state_slots,
+                const Tensor& context_lens, const Tensor& query_start, Tensor& out, bool silu) {
+  vgate::ShortConvArgs p;
+  p.f32 = act_f32(x, "x");
+  TORCH_CHECK(x.dim() == 2 && out.dim() == 2 && act_f32(out, "out") == p.f32 && out.size(0) <= x.size(0) && out.size(1) == x.size(1),
+              "short_conv: x, out [T, C] of one dtype");
+  p.T = (int)out.size(0); p.C = (int)x.size(1);
+  TORCH_CHECK(w.dim() == 2 && w.size(0) >= 1 && w.size(0) <= 4096 && w.size(1) == p.C, "short_conv: w [taps, C]");
+  p.taps = (int)w.size(0);
+  OptT wo(w);
+  p.w = f32p(wo, "w", (int64_t)p.taps * p.C); p.b = f32p(b, "b", p.C);
+  p.kept = kept_rows(kept, p.taps, p.C);
+  p.x = x.data_ptr(); p.ldx = x.stride(0); p.out = out.data_ptr(); p.ldo = out.stride(0);
+  p.act = silu ? 1 : 0;
+  p.S = (int)state_slots.numel();
+  p.state_slots = slots_of(state_slots, p.S);
+  p.context_lens = i32p(context_lens, "context_lens", p.S);
+  p.query_start = i32p(query_start, "query_start", p.S + 1);  // values <= T: set by the step metadata
+  c10::DeviceGuard guard(x.device());
+  vgate::launch_short_conv(p, cur_stream());
+}
+
+// x, z, xin [T, C] (activation dtype), dt fp32 [T, C], B, C [T, N] with one row stride; A [C, N] times log2(e)
+void selective_scan(const Tensor& x, const Tensor& dt, const Tensor& B, const Tensor& Cm, const Tensor& z, const Tensor& A,
+                    const Tensor& D, const Tensor& xin, Tensor& state, Tensor& kept, const Tensor& state_slots,
+                    const Tensor& context_lens, const Tensor& query_start, Tensor& out, Tensor& scratch) {
+  vgate::SelectiveScanArgs p;
+  p.f32 = act_f32(x, "x");
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == torch::kFloat32 && state.is_contiguous() && state.dim() == 3,
+              "selective_scan: state fp32 [slots, C, N]");
+  p.C = (int)state.size(1); p.N = (int)state.size(2);
+  TORCH_CHECK(p.N >= 1 && p.N <= 256, "selective_scan: 1..256 states per channel");
+  const int64_t T = x.size(0);
+  auto rows = [&](const Tensor& t, int64_t n, const char* name) {
+    TORCH_CHECK(act_f32(t, name) == p.f32 && t.dim() == 2 && t.size(0) == T && t.size(1) == n, "selective_scan: ", name, " [T, ", n, "]");
+  };
+  rows(x, p.C, "x"); rows(z, p.C, "z"); rows(xin, p.C, "xin"); rows(out, p.C, "out"); rows(B, p.N, "B"); rows(Cm, p.N, "C");
+  TORCH_CHECK(B.stride(0) == Cm.stride(0), "selective_scan: B and C share a row stride");
+  TORCH_CHECK(dt.is_cuda() && dt.scalar_type() == torch::kFloat32 && dt.dim() == 2 && dt.stride(1) == 1 && dt.size(0) == T &&
+              dt.size(1) == p.C, "selective_scan: dt fp32 [T, C]");
+  p.x = x.data_ptr(); p.ldx = x.stride(0); p.z = z.data_ptr(); p.ldz = z.stride(0); p.xin = xin.data_ptr(); p.ldxin = xin.stride(0);
+  p.B = B.data_ptr(); p.Cm = Cm.data_ptr(); p.ldbc = B.stride(0); p.dt = dt.data_ptr<float>(); p.lddt = dt.stride(0);
+  p.out = out.data_ptr(); p.ldo = out.stride(0);
+  OptT o0(A), o1(D);
+  p.A = f32p(o0, "A", (int64_t)p.C * p.N); p.D = f32p(o1, "D", p.C);
+  TORCH_CHECK(kept.dim() == 3 && kept.size(0) == state.size(0), "selective_scan: kept [slots, taps - 1, C]");
+  p.taps = (int)kept.size(1) + 1;
+  p.kept = const_cast<float*>(kept_rows(kept, p.taps, p.C));
+  p.state = state.data_ptr<float>();
+  p.S = (int)state_slots.numel();
+  p.state_slots = slots_of(state_slots, p.S);
+  p.context_lens = i32p(context_lens, "context_lens", p.S);
+  p.query_start = i32p(query_start, "query_start", p.S + 1);
+  TORCH_CHECK(scratch.is_cuda() && scratch.scalar_type() == torch::kFloat32 && scratch.is_contiguous() &&
+              (size_t)scratch.numel() >= vgate::selective_scan_scratch_floats((int)T, p.S, p.C, p.N),
+              "selective_scan: scratch fp32 with selective_scan_scratch(T, S, C, N) elements");
+  c10::DeviceGuard guard(x.device());
+  vgate::launch_selective_scan(p, (int)T, scratch.data_ptr<float>(), cur_stream());
 }
 
 void moe_route(const Tensor& z, const OptT& corr, int64_t top, double norm_eps, Tensor& idx, Tensor& wts, int64_t score,
@@ -750,8 +913,10 @@ void bind_seq(pybind11::module& m) {
         py::arg("g2") = py::none(), py::arg("b2") = py::none());
   m.def("latent_write", &latent_write, "latent norm + shared-key rotation + paged cache store", py::arg("kv"), py::arg("w"),
         py::arg("eps"), py::arg("positions"), py::arg("slots"), py::arg("inv_freq"), py::arg("rot_dims"), py::arg("cache"),
-        py::arg("rank"), py::arg("cache_t") = py::none());
-  m.def("latent_qrope", &latent_qrope, "rotate the rotated query part into the absorbed query buffer");
+        py::arg("rank"), py::arg("cache_t") = py::none(), py::arg("rot_half") = false, py::arg("rot_amp") = 1.0);
+  m.def("latent_qrope", &latent_qrope, "rotate the rotated query part into the absorbed query buffer", py::arg("q"),
+        py::arg("positions"), py::arg("inv_freq"), py::arg("rot_dims"), py::arg("qa"), py::arg("H"), py::arg("dim"),
+        py::arg("rank"), py::arg("rot"), py::arg("rot_half") = false, py::arg("rot_amp") = 1.0);
   m.def("latent_attn", &latent_attn, "causal attention over the paged latent cache (absorbed projections)", py::arg("qa"),
         py::arg("cache"), py::arg("block_tables"), py::arg("context_lens"), py::arg("query_start"), py::arg("ol"),
         py::arg("scale"), py::arg("H"), py::arg("rank"), py::arg("rot"), py::arg("cache_t") = py::none(),
@@ -772,6 +937,20 @@ void bind_seq(pybind11::module& m) {
         py::arg("x"), py::arg("y"), py::arg("mult"), py::arg("w") = py::none(), py::arg("eps") = 0.0,
         py::arg("h_out") = py::none(), py::arg("post_w") = py::none(), py::arg("center") = false, py::arg("pos") = py::none(),
         py::arg("wts") = py::none());
+  m.def("branch_residual", &branch_residual,
+        "x += s1 (normed) y1 + s2 (normed) y2 + y3 in fp32, and the new rows' norm under one or two weights", py::arg("x"),
+        py::arg("y1"), py::arg("s1"), py::arg("w1"), py::arg("y2"), py::arg("s2"), py::arg("w2"), py::arg("y3"), py::arg("eps"),
+        py::arg("n1"), py::arg("h1"), py::arg("n2"), py::arg("h2"), py::arg("T"));
+  m.def("gated_delta", &gated_delta, "gated delta rule recurrence over state slots behind short convolutions + head norm + gate",
+        py::arg("q"), py::arg("k"), py::arg("v"), py::arg("b"), py::arg("z"), py::arg("gate"), py::arg("decay"), py::arg("nw"),
+        py::arg("conv_w"), py::arg("state"), py::arg("conv_state"), py::arg("state_slots"), py::arg("context_lens"),
+        py::arg("query_start"), py::arg("out"), py::arg("unit_eps"), py::arg("q_scale"), py::arg("eps"), py::arg("scratch"),
+        py::arg("wide") = -1);
+  m.def("short_conv", &short_conv, "short causal convolution over time per channel (+ silu) over state slots");
+  m.def("selective_scan_scratch", [](int64_t T, int64_t S, int64_t C, int64_t N) {
+    return (int64_t)vgate::selective_scan_scratch_floats((int)T, (int)S, (int)C, (int)N);
+  }, "fp32 elements of scratch a selective_scan call over T rows and S sequences needs");
+  m.def("selective_scan", &selective_scan, "selective scan over state slots + D x + silu gate; keeps the convolution's inputs");
   m.def("pair_rows", &pair_rows, "two fp32 row sets side by side in the activation dtype");
   m.def("shift_mix", &shift_mix, "blends of every token's row with the row of the token before it; keeps the last row");
   m.def("map_pair_combine", &map_pair_combine, "two attention maps per head: a1 - lam a2, head RMS norm, scale, gate");
@@ -791,10 +970,12 @@ void bind_seq(pybind11::module& m) {
         py::arg("query_start"), py::arg("out"), py::arg("scale"), py::arg("H"), py::arg("window"), py::arg("pool"),
         py::arg("sink"), py::arg("v_freq"), py::arg("vt") = py::none(), py::arg("prefill_kernel") = 0,
         py::arg("bias_kind") = 0, py::arg("bias_a") = py::none(), py::arg("bias_b") = py::none(), py::arg("gate") = py::none(),
-        py::arg("parts") = 1, py::arg("part_scratch") = py::none(), py::arg("softcap") = 0.0, py::arg("chunk") = 0);
+        py::arg("parts") = 1, py::arg("part_scratch") = py::none(), py::arg("softcap") = 0.0, py::arg("chunk") = 0,
+        py::arg("keep") = 0);
   m.def("window_attn_split", [](int64_t T, int64_t S, int64_t H, int64_t G, int64_t D, int64_t V, bool f32, int64_t page,
-                                int64_t chunk) {
-    const int parts = vgate::window_attn_parts((int)T, (int)S, (int)H, (int)G, (int)D, (int)V, f32 ? 1 : 0, (int)page, (int)chunk);
+                                int64_t window, int64_t chunk, int64_t keep, int64_t pool) {
+    const int parts = vgate::window_attn_parts((int)T, (int)S, (int)H, (int)G, (int)D, (int)V, f32 ? 1 : 0, (int)page,
+                                               vgate::window_attn_span((int)window, (int)chunk, (int)keep, (int)pool));
     return std::make_pair((int64_t)parts, (int64_t)vgate::window_attn_part_floats((int)T, (int)S, (int)H, (int)G, (int)D, (int)V, parts));
   }, "workgroups that share a decoded token's key tiles in window_attn, and the fp32 scratch elements they need");
   m.def("linear_attn_scratch", [](int64_t T, int64_t S, int64_t H, int64_t D, int64_t V) {

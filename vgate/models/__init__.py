@@ -4,7 +4,7 @@ from __future__ import annotations
 # family (ModelArch.family / HybridArch.family) -> model class, imported on first use
 TRANSFORMER_FAMILIES = {"qwen2", "llama"}   # vgate.models.transformer.DecoderModel
 # vgate.models.hybrid.HybridModel (layered: mixers + feed-forwards)
-HYBRID_FAMILIES = {"zadirax", "pozalorn", "livitar", "gefudra", "nigozen"}
+HYBRID_FAMILIES = {"zadirax", "pozalorn", "livitar", "gefudra", "nigozen", "vugudra"}
 
 
 def build_model(arch, device, tp=None, quantization=None, seed: int = 0, weights_path: str | None = None,

@@ -156,9 +156,10 @@ class HybridArch:
     norm: str = "rms"
     embed_scale: float = 1.0
     # (start, stop, times): layers start .. stop - 1 run ``times`` times in a row with the same weights, every
-    # pass with caches and states of its own; right before the first layer of each pass the stream is replaced by
-    # W_in [x; x0] (tensor ``loop.in`` [width, 2 width], x0 the embedding output)
+    # pass with caches and states of its own; with ``loop_input`` the stream is replaced by W_in [x; x0] (tensor
+    # ``loop.in`` [width, 2 width], x0 the embedding output) right before the first layer of each pass
     loop: tuple | None = None
+    loop_input: bool = True
     # the logits are multiplied by this; with ``tie_embeddings`` the embedding table is the output matrix
     logit_scale: float = 1.0
     tie_embeddings: bool = False
@@ -320,6 +321,17 @@ def _livitar_from_config(cfg: dict, name: str) -> HybridArch:
                       arrangement="hyper_pre_norm", streams=streams)
 
 
+def _loop_from_config(cfg: dict, layers: int) -> tuple | None:
+    """(start, stop, times) of config.json's ``loop`` (None: absent or an empty stretch)."""
+    lp = cfg.get("loop")
+    if not lp:
+        return None
+    a, b, times = int(lp["start"]), int(lp["stop"]), int(lp["times"])
+    if not (0 <= a <= b <= layers) or times < 0:
+        raise ValueError("loop: 0 <= start <= stop <= layers, times >= 0")
+    return (a, b, times) if b > a else None
+
+
 def _gefudra_mixer(kind: str, m: dict) -> tuple:
     """(key of ``vgate.models.mixers.MIXERS``, its spec) of a Gefudra layer type. What the design fixes (no
     rotated key part, which gate, which norm, the two score maps) is written out here as options of the mixers."""
@@ -353,14 +365,7 @@ def _gefudra_from_config(cfg: dict, name: str) -> HybridArch:
                 raise ValueError(f"Gefudra feed-forward kind {mlp.get('kind')!r}")
             mlp = {"kind": "dense", "ff": int(mlp["ff"]), "act": "clamped", "limit": float(mlp["limit"])}
         layers.append(LayerSpec(kind=kind, mixer=spec, mlp=mlp or None))
-    loop = None
-    lp = cfg.get("loop")
-    if lp:
-        a, b, times = int(lp["start"]), int(lp["stop"]), int(lp["times"])
-        if not (0 <= a <= b <= len(layers)) or times < 0:
-            raise ValueError("loop: 0 <= start <= stop <= layers, times >= 0")
-        if b > a:
-            loop = (a, b, times)
+    loop = _loop_from_config(cfg, len(layers))
     eos = cfg.get("eos_token_id", 2)
     return HybridArch(name=name, family="gefudra", hidden_size=int(cfg["width"]), vocab_size=int(cfg["vocab"]),
                       layers=tuple(layers), rms_eps=float(cfg["norm"]["eps"]), bos_token_id=int(cfg.get("bos_token_id", 1)),
@@ -410,9 +415,54 @@ def _nigozen_from_config(cfg: dict, name: str) -> HybridArch:
                       norm="layer", embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), tie_embeddings=True)
 
 
+def _vugudra_mixer(kind: str, m: dict) -> tuple:
+    """(key of ``vgate.models.mixers.MIXERS``, its spec) of a Vugudra layer type. What the design fixes (which pairs a
+    rotation turns, one gate per head, keys that are also the values, the normed half-and-half sum) is written out here
+    as options of the mixers."""
+    if kind == "latent_attention":   # keys / values from a cached low-rank row + one shared rotated key part; sink; head gate
+        rot = m["rot"]
+        return "latent_attention", {"heads": int(m["heads"]), "dim": int(m["dim"]), "rot_dim": int(m["rot_dim"]),
+                                    "vdim": int(m["vdim"]), "kv_rank": int(m["kv_rank"]), "q_rank": int(m["q_rank"]),
+                                    "scale": float(m["scale"]), "sink": True, "gate": "head", "out_f32": True,
+                                    "rot": {"dims": int(rot["dims"]), "base": float(rot["base"]), "layout": "half",
+                                            "scaling": dict(rot["scaling"]) if rot.get("scaling") else None}}
+    if kind == "parallel":           # window attention over keys that are the values, beside a gated delta rule
+        a, r = m["left"], m["right"]
+        rot, mask = a["rot"], a["mask"]
+        left = {"heads": int(a["heads"]), "kv_heads": int(a["kv_heads"]), "dim": int(a["dim"]), "vdim": int(a["vdim"]),
+                "scale": float(a["scale"]), "window": int(mask["size"]), "keep_first": int(mask.get("keep_first") or 0),
+                "values": "keys", "qk_norm": "head",
+                "rot": {"dims": int(rot["dims"]), "base": float(rot["base"]), "layout": "pairs"}}
+        right = {n: int(r[n]) for n in ("heads", "kv_heads", "dim", "vdim", "conv")}
+        return "parallel", {"left": ("window_attention", left), "right": ("gated_delta", right), "left_scale": 0.5,
+                            "right_scale": 0.5, "out_norm": True}
+    if kind == "mamba1":             # selective scan behind a short convolution
+        return "mamba1", {n: int(m[n]) for n in ("inner", "state", "dt_rank", "conv")}
+    raise ValueError(f"Vugudra has no layer type {kind!r}")
+
+
+def _vugudra_from_config(cfg: dict, name: str) -> HybridArch:
+    """config.json of the Vugudra design: layers whose mixer and feed-forward read the same stream through two norms
+    (weights around zero), a stretch of layers that runs several times with the same weights, an output matrix of its own."""
+    layers = []
+    for L in cfg["layers"]:
+        kind, spec = _vugudra_mixer(L["type"], L["mixer"])
+        mlp = L.get("mlp")
+        if mlp:
+            if mlp.get("kind") != "dense":
+                raise ValueError(f"Vugudra feed-forward kind {mlp.get('kind')!r}")
+            mlp = {"kind": "dense", "ff": int(mlp["ff"]), "act": "silu"}
+        layers.append(LayerSpec(kind=kind, mixer=spec, mlp=mlp or None))
+    eos = cfg.get("eos_token_id", 2)
+    return HybridArch(name=name, family="vugudra", hidden_size=int(cfg["width"]), vocab_size=int(cfg["vocab"]),
+                      layers=tuple(layers), rms_eps=float(cfg["norm"]["eps"]), bos_token_id=int(cfg.get("bos_token_id", 1)),
+                      eos_token_ids=tuple(eos) if isinstance(eos, list) else (int(eos),), arrangement="parallel_norm",
+                      loop=_loop_from_config(cfg, len(layers)), loop_input=False)
+
+
 # config.json "architecture" -> parser of a layered hybrid design
 HYBRID_ARCHITECTURES = {"Zadirax": _zadirax_from_config, "Pozalorn": _pozalorn_from_config, "Livitar": _livitar_from_config,
-                        "Gefudra": _gefudra_from_config, "Nigozen": _nigozen_from_config}
+                        "Gefudra": _gefudra_from_config, "Nigozen": _nigozen_from_config, "Vugudra": _vugudra_from_config}
 
 
 def _zadirax_preset(name: str, width: int, vocab: int, pairs: int, heads: int, dim: int, ff: int, experts: int,
@@ -503,6 +553,27 @@ def _nigozen_preset(name: str, width: int, vocab: int, heads: int, kv_heads: int
     return _nigozen_from_config(cfg, name)
 
 
+def _vugudra_preset(name: str, width: int, vocab: int, groups: int, heads: int, kv_heads: int, dim: int, ff: int, kv_rank: int,
+                    q_rank: int, rot: int, window: int, keep: int, inner: int, state: int, dt_rank: int, conv: int = 4,
+                    loop_times: int = 0) -> HybridArch:
+    """Random-init Vugudra models (benchmarks, tests): ``groups`` x [latent attention, window attention beside a gated
+    delta rule, selective scan], the first group's last two layers looped ``loop_times`` times."""
+    mlp = {"kind": "dense", "ff": ff}
+    lat = {"type": "latent_attention", "mlp": mlp,
+           "mixer": {"heads": heads, "dim": dim, "vdim": dim, "kv_rank": kv_rank, "q_rank": q_rank, "rot_dim": rot,
+                     "scale": (dim + rot) ** -0.5,
+                     "rot": {"base": 10000.0, "dims": rot, "scaling": {"factor": 4.0, "original": 4096, "fast": 32, "slow": 1}}}}
+    par = {"type": "parallel", "mlp": mlp,
+           "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                              "rot": {"base": 10000.0, "dims": dim}, "mask": {"size": window, "keep_first": keep}},
+                     "right": {"heads": heads, "kv_heads": heads, "dim": dim, "vdim": dim, "conv": conv}}}
+    mam = {"type": "mamba1", "mlp": mlp, "mixer": {"inner": inner, "state": state, "dt_rank": dt_rank, "conv": conv}}
+    cfg = {"width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "layers": [lat, par, mam] * groups}
+    if loop_times > 0:
+        cfg["loop"] = {"start": 1, "stop": 3, "times": loop_times}
+    return _vugudra_from_config(cfg, name)
+
+
 HYBRID_PRESETS = {
     # tests / CPU smoke: odd sizes on purpose (nothing a multiple of the MFMA tile)
     "zadirax-tiny": lambda: _zadirax_preset("zadirax-tiny", 96, 300, 2, 3, 24, 136, 5, 2, 40, 56, 40, 8, share=True),
@@ -537,6 +608,14 @@ HYBRID_PRESETS = {
     # of the other bench presets
     "nigozen-bench-1024": lambda: _nigozen_preset("nigozen-bench-1024", 1024, 32000, 8, 2, 128, 128, 64, 1024, 6144, 8, 2, 3072),
     "nigozen-bench-1536": lambda: _nigozen_preset("nigozen-bench-1536", 1536, 32000, 12, 2, 128, 128, 64, 1024, 13440, 16, 4, 3328),
+    # tests / CPU smoke: odd sizes on purpose
+    "vugudra-tiny": lambda: _vugudra_preset("vugudra-tiny", 88, 300, 1, 4, 2, 24, 136, 40, 56, 10, 21, 3, 100, 6, 7, loop_times=2),
+    # slices at the layer sizes of real models beside a transformer of equal width (benchmarks/design_compare.py): three
+    # layers, each run once
+    "vugudra-bench-1024": lambda: _vugudra_preset("vugudra-bench-1024", 1024, 32000, 1, 8, 2, 128, 4096, 256, 512, 64, 1024, 64,
+                                                  2048, 16, 64),
+    "vugudra-bench-1536": lambda: _vugudra_preset("vugudra-bench-1536", 1536, 32000, 1, 12, 2, 128, 8960, 512, 768, 64, 1024, 64,
+                                                  3072, 16, 96),
     # layer sizes of a ~1.5B model (the width, head size, feed-forward and vocabulary of qwen2.5-1.5b)
     "zadirax-1.5b": lambda: _zadirax_preset("zadirax-1.5b", 1536, 151936, 14, 12, 128, 8960, 32, 4, 2240, 512, 768, 64),
 }

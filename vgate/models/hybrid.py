@@ -22,11 +22,13 @@ Layer arrangements (``ARRANGEMENTS``, chosen by ``HybridArch.arrangement``):
   sandwich_norm   x += m * norm1b(mixer(norm1(x)));  x += m * norm2b(ff(norm2(x))): a norm before and after each sublayer
                   (a sublayer's output norm, its add and the next sublayer's norm are one kernel, which for a mixture
                   of experts also sums a token's weighted expert rows)
-The norms of the last two are RMS or layer norms (``HybridArch.norm``); the embedding rows may be scaled
+  parallel_norm   x += mixer(rmsnorm(x) (1 + w1)) + ff(rmsnorm(x) (1 + w2)): both sublayers read the same stream (a layer's
+                  add and both norms of the next layer are one kernel)
+The norms of the pre_norm and sandwich_norm arrangements are RMS or layer norms (``HybridArch.norm``); the embedding rows may be scaled
 (``HybridArch.embed_scale``).
 ``HybridArch.loop`` = (start, stop, times): the layers start .. stop - 1 run ``times`` times in a row with the same
-weights, every pass with caches and states of its own; right before the first layer of each pass the stream
-becomes W_in [x; x0] (``loop.in``, x0 the embedding output).
+weights, every pass with caches and states of its own; with ``HybridArch.loop_input`` the stream becomes W_in [x; x0] (``loop.in``,
+x0 the embedding output) right before the first layer of each pass.
 With ``HybridArch.depth_average`` the stream a layer hands on is a learned combination of the
 embedding output X_0 and every layer result X_1 .. X_(i+1): sum_j c_i[j] X_j (tensor ``l<i>.dwa``).
 A layer may run with another layer's weights (``weights_of``) while keeping its own cache or state.
@@ -129,6 +131,8 @@ class PostNormLayer:
         mix = {k[4:]: v for k, v in t.items() if k.startswith("mix.")}
         self.eps = eps
         self.mixer = MIXERS[spec.kind](spec.mixer, width, eps, mix, device, f32)
+        if getattr(self.mixer, "out_norms", None):
+            raise ValueError("the post_norm arrangement norms the sum of two mixers, not each of them")
         self.norm1 = _f32(t["norm1"], device)
         self.ff = self.norm2 = None
         if spec.mlp:
@@ -317,19 +321,70 @@ class SandwichNormLayer(PreNormLayer):
         return out
 
 
-class _PreStream:
-    """The stream of one ``pre_norm`` or ``sandwich_norm`` step: ``x`` fp32 [T, W], ``h`` the next sublayer's normed
-    input, ``carry`` what the mixers of the step's layer runs hand on to each other."""
+class ParallelNormLayer:
+    """``parallel_norm`` arrangement: x += mixer(rmsnorm(x) (1 + norm1)) + ff(rmsnorm(x) (1 + norm2)), both of the same x.
+    The residual kernel adds the sublayers' results (two mixers side by side: each normed and scaled first) and makes
+    both normed inputs of the layer that follows from one set of statistics."""
 
-    def __init__(self, T: int, W: int, act_dtype, device):
+    carries = False
+
+    def __init__(self, spec, width: int, eps: float, t: dict, device, f32: bool):
+        mix = {k[4:]: v for k, v in t.items() if k.startswith("mix.")}
+        self.eps = eps
+        self.mixer = MIXERS[spec.kind](spec.mixer, width, eps, mix, device, f32)
+        self.norm1 = 1.0 + _f32(t["norm1"], device)
+        self.ff = self.norm2 = None
+        if spec.mlp:
+            mlp = {k[4:]: v for k, v in t.items() if k.startswith("mlp.")}
+            self.ff = FEED_FORWARDS[spec.mlp["kind"]](spec.mlp, width, mlp, device, f32)
+            self.norm2 = 1.0 + _f32(t["norm2"], device)
+        self.proj, self.col = _fuse_inputs(self.mixer, [], width, device, f32)
+
+    shapes = staticmethod(PreNormLayer.shapes)
+
+    def cols(self, P: torch.Tensor, name: str) -> torch.Tensor:
+        a, n = self.col[name]
+        return P[:, a: a + n]
+
+    def nbytes(self) -> int:
+        return (self.proj.nbytes() if self.proj else 0) + self.mixer.nbytes() + (self.ff.nbytes() if self.ff else 0)
+
+    def inputs(self, st) -> list:
+        """What the kernel before this layer makes: its sublayers' normed inputs."""
+        return [(self.norm1, st.h)] + ([(self.norm2, st.h2)] if self.ff is not None else [])
+
+    def run(self, st, sv, cache) -> None:
+        """st.x: the fp32 stream; st.h, st.h2: the normed inputs in the activation dtype (``st.h_ready``: made by the kernel
+        before); st.next_layer: the layer that follows, or None."""
+        if not st.h_ready:
+            seq.branch_residual(st.x, [], self.eps, outs=self.inputs(st))
+        P = self.proj(st.h) if self.proj is not None else None
+        y = self.mixer.forward(st.h, P, self.cols, sv, cache)
+        if isinstance(y, tuple):
+            w = getattr(self.mixer, "out_norms", None) or (None, None)
+            ys = [(y[0], y[1], w[0]), (y[2], y[3], w[1])]
+        else:
+            ys = [(y, 1.0, None)]
+        yf = self.ff.forward(st.h2, out_f32=True) if self.ff is not None else None
+        nxt = st.next_layer
+        seq.branch_residual(st.x, ys, self.eps, y3=yf, outs=nxt.inputs(st) if nxt is not None else None)
+        st.h_ready = nxt is not None
+
+
+class _PreStream:
+    """The stream of one ``pre_norm``, ``sandwich_norm`` or ``parallel_norm`` step: ``x`` fp32 [T, W], ``h`` (and ``h2``) the
+    next sublayers' normed input, ``carry`` what the mixers of the step's layer runs hand on to each other."""
+
+    def __init__(self, T: int, W: int, act_dtype, device, second: bool = False):
         self.x = torch.empty(T, W, dtype=torch.float32, device=device)
         self.h = torch.empty(T, W, dtype=act_dtype, device=device)
-        self.h_ready, self.next_norm = False, None
+        self.h2 = torch.empty_like(self.h) if second else None
+        self.h_ready, self.next_norm, self.next_layer = False, None, None
         self.carry: dict = {}
 
 
 ARRANGEMENTS = {"gated_parallel": GatedParallelLayer, "post_norm": PostNormLayer, "hyper_pre_norm": HyperPreNormLayer,
-                "pre_norm": PreNormLayer, "sandwich_norm": SandwichNormLayer}
+                "pre_norm": PreNormLayer, "sandwich_norm": SandwichNormLayer, "parallel_norm": ParallelNormLayer}
 
 
 class _HyperStream:
@@ -406,8 +461,11 @@ class HybridModel:
         tensors = load_tensors(arch, weights_path) if weights_path else random_tensors(arch, seed)
         self.embed = tensors["embed"].to(self.device, self.act_dtype).contiguous()
         layer_cls = ARRANGEMENTS[arch.arrangement]
-        self.pre = arch.arrangement in ("pre_norm", "sandwich_norm")
-        extra = {"mult": arch.residual_mult, "norm": arch.norm} if self.pre else {}
+        self.side = arch.arrangement == "parallel_norm"
+        self.pre = arch.arrangement in ("pre_norm", "sandwich_norm") or self.side
+        extra = {"mult": arch.residual_mult, "norm": arch.norm} if self.pre and not self.side else {}
+        if self.side and (arch.norm != "rms" or arch.residual_mult != 1.0):
+            raise ValueError("the parallel_norm arrangement has RMS norms and no residual multiplier")
         if not self.pre and (arch.norm != "rms" or arch.embed_scale != 1.0):
             raise ValueError(f"layer norms and scaled embeddings need the pre_norm or sandwich_norm arrangement, not {arch.arrangement}")
         owned: dict = {}
@@ -429,14 +487,16 @@ class HybridModel:
         if len({L.mixer.G * L.mixer.V for L in owned.values() if getattr(L.mixer, "value_mix", False)}) > 1:
             raise ValueError("layers that mix values need the same kv_heads * vdim")
         self._owned = owned
-        self.loop_in = Proj(tensors["loop.in"], self.device, self.f32) if arch.loop is not None else None
+        if arch.loop is not None and not self.pre:
+            raise ValueError(f"looped layers need the pre_norm, sandwich_norm or parallel_norm arrangement, not {arch.arrangement}")
+        self.loop_in = Proj(tensors["loop.in"], self.device, self.f32) if arch.loop is not None and arch.loop_input else None
         # depth-average coefficients belong to the position in the stack, not to the (possibly shared) weights
         self.depth_coef = [_f32(tensors[f"l{i}.dwa"], self.device) for i in range(arch.num_layers)] \
             if arch.depth_average else None
         self.scalar_norm = arch.arrangement == "gated_parallel"   # one number per norm, or a weight vector
         self.hyper = arch.arrangement == "hyper_pre_norm"
         self.final_norm = _TanhNorm(tensors, "final.norm", self.device) if self.hyper else \
-            _f32(tensors["final.norm"].reshape(-1), self.device)
+            _f32(tensors["final.norm"].reshape(-1), self.device) + (1.0 if self.side else 0.0)
         if arch.logit_scale != 1.0:   # logits = head (norm(x) w) s = head (norm(x) (w s)): one fp32 product, made here
             if self.hyper:
                 raise ValueError("a logit scale needs an RMS final norm")
@@ -505,10 +565,10 @@ class HybridModel:
         return st.x
 
     def _forward_pre(self, sv, caches) -> torch.Tensor:
-        """The layer loop of the ``pre_norm`` and ``sandwich_norm`` arrangements, with the looped stretch; returns the
-        fp32 stream."""
+        """The layer loop of the ``pre_norm``, ``sandwich_norm`` and ``parallel_norm`` arrangements, with the looped stretch;
+        returns the fp32 stream."""
         T, W = sv.T, self.arch.hidden_size
-        st = _PreStream(T, W, self.act_dtype, self.device)
+        st = _PreStream(T, W, self.act_dtype, self.device, second=self.side)
         seq.embed_rows(sv.ids, self.embed, st.x, prev=sv.prev_tokens, scale=self.arch.embed_scale)
         x0 = pair = None
         if self.loop_in is not None:
@@ -516,12 +576,12 @@ class HybridModel:
             pair = torch.empty(T, 2 * W, dtype=self.act_dtype, device=self.device)
         n = len(self.layers)
         for ri, L in enumerate(self.layers):
-            if self.pass_start[ri]:   # x <- W_in [x; x0]
+            if self.loop_in is not None and self.pass_start[ri]:   # x <- W_in [x; x0]
                 seq.pair_rows(st.x, x0, pair)
                 self.loop_in(pair, out_f32=True, out=st.x)
                 st.h_ready = False
-            nxt = self.layers[ri + 1] if ri + 1 < n and not self.pass_start[ri + 1] else None
-            st.next_norm = nxt.norm1 if nxt is not None else None
+            nxt = self.layers[ri + 1] if ri + 1 < n and not (self.loop_in is not None and self.pass_start[ri + 1]) else None
+            st.next_layer, st.next_norm = nxt, nxt.norm1 if nxt is not None else None
             L.run(st, sv, caches[ri])
             if self.capture_layers is not None:
                 self.capture_layers.append(st.x.clone())
@@ -559,7 +619,7 @@ def tensor_shapes(arch: HybridArch, nominal: int | None = 16) -> dict:
     out = {"embed": (arch.vocab_size, W), "final.norm": (W,) if vector else ()}
     if not arch.tie_embeddings:
         out["head"] = (arch.vocab_size, W)
-    if arch.loop is not None:
+    if arch.loop is not None and arch.loop_input:
         out["loop.in"] = (W, 2 * W)
     extra = {}
     if arch.arrangement == "hyper_pre_norm":
@@ -629,8 +689,9 @@ def random_tensors(arch: HybridArch, seed: int = 0) -> dict:
             w = torch.randn(shape, generator=g) * std
         elif leaf == "vmix":             # a blend weight between two layers' values
             w = 0.2 + 0.6 * torch.rand(shape, generator=g)
-        elif leaf in ("norm", "norm1", "norm2", "norm1b", "norm2b") or name == "final.norm":
-            w = 1.0 + 0.1 * torch.randn(shape, generator=g)
+        elif leaf in ("norm", "norm1", "norm2", "norm1b", "norm2b") or name == "final.norm" or (leaf == "out" and not hyper):
+            around_zero = arch.arrangement == "parallel_norm" and (leaf in ("norm1", "norm2") or name == "final.norm")
+            w = (0.0 if around_zero else 1.0) + 0.1 * torch.randn(shape, generator=g)
         else:
             w = 0.3 * torch.randn(shape, generator=g)
         out[name] = w.to(torch.bfloat16)

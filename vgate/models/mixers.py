@@ -22,7 +22,11 @@ spec, so another design can reuse a mixer with other values.
 * :class:`ShiftedLinearAttention` — the same kind of recurrence read before its update, with a bonus on the
   current token's own outer product, a decay exp(-exp(.)) per key channel from a low-rank gate, and every
   projection reading its own blend of the token's and the previous token's input (which is part of the state).
-* :class:`ParallelMixers` — two mixers reading the same input, their outputs added with fixed scales.
+* :class:`GatedDelta` — delta rule with one decay per head and key channel, unit-norm keys and queries behind a short
+  causal convolution, over an fp32 state per head; the convolution's last inputs are state too.
+* :class:`SelectiveScan` — diagonal recurrence per (channel, state) with an input-dependent step behind a short causal
+  convolution, gated by the other half of its input projection.
+* :class:`ParallelMixers` — two mixers reading the same input, their outputs (optionally each normed) added with fixed scales.
 * :class:`DenseFF`, :class:`MoEFF` — feed-forward (gated pair, or one matrix and an activation); mixture of such
   experts (sigmoid scores with a selection-only correction, softmax scores over all experts or over the chosen,
   optional shared expert).
@@ -107,7 +111,9 @@ def _pad8(w: torch.Tensor) -> torch.Tensor:
 # ------------------------------------------------------------------------------------------ mixers
 class LatentAttention:
     """Attention through a low-rank key/value latent. spec: heads, dim, vdim, kv_rank, q_rank, scale, ``rot_dim``
-    (size of the rotated key part all heads share; 0: none) with ``rot`` {dims, base}, and the options ``window``
+    (size of the rotated key part all heads share; 0: none) with ``rot`` {dims, base, layout "pairs" (entry 2i with
+    2i + 1, the default) or "half" (entry i with i + dims / 2), scaling (:func:`vgate.ops.seq.rope_inv_freq`)}, and the
+    options ``gate`` "channel" (W_g has a row per head and value channel, the default) or "head" (one per head), ``window``
     (position i sees j with 0 <= i - j < window; None: every earlier position), ``sink`` (one learned logit per
     head, tensor ``sink``, that only enters the softmax denominator), ``out_f32`` (the output projection writes
     fp32 for an fp32 residual sum)."""
@@ -130,11 +136,15 @@ class LatentAttention:
         if dims > self.R or dims < 0:
             raise ValueError("latent_attention: rot.dims must be <= rot_dim")
         self.rot_dims = 2 * (dims // 2)  # entries in rotated pairs (an odd last one passes unchanged)
+        if rot.get("layout", "pairs") not in ("pairs", "half") or m.get("gate", "channel") not in ("channel", "head"):
+            raise ValueError("latent_attention: rot.layout pairs | half, gate channel | head")
+        self.rot = {"rot_half": rot.get("layout", "pairs") == "half", "rot_amp": seq.rope_amplitude(rot.get("scaling"))}
+        self.head_gate = m.get("gate", "channel") == "head"
         self.eps = eps
         self.f32 = f32
         dev = torch.device(device)
         H, D, R, V, KR = self.H, self.D, self.R, self.V, self.KR
-        self.inv_freq = seq.rope_inv_freq(dims, float(rot.get("base", 10000.0)), dev)  # base^(-2i / dims)
+        self.inv_freq = seq.rope_inv_freq(dims, float(rot.get("base", 10000.0)), dev, scaling=rot.get("scaling"))
         self.in_rows = [("dq", tensors["dq"]), ("dkv", tensors["dkv"]), ("g", tensors["g"])]
         self.in_bias = {}
         self.dq_norm, self.dkv_norm = _f32(tensors["dq.norm"], dev), _f32(tensors["dkv.norm"], dev)
@@ -151,7 +161,8 @@ class LatentAttention:
         H, D, R, V = spec["heads"], spec["dim"], spec.get("rot_dim", 0), spec["vdim"]
         KR, QR = spec["kv_rank"], spec["q_rank"]
         out = {"dq": (QR, width), "dq.norm": (QR,), "uq": (H * (D + R), QR), "dkv": (KR + R, width),
-               "dkv.norm": (KR,), "uk": (H * D, KR), "uv": (H * V, KR), "g": (H * V, width), "o": (width, H * V)}
+               "dkv.norm": (KR,), "uk": (H * D, KR), "uv": (H * V, KR),
+               "g": (H if spec.get("gate") == "head" else H * V, width), "o": (width, H * V)}
         if spec.get("sink"):
             out["sink"] = (H,)
         return out
@@ -192,16 +203,17 @@ class LatentAttention:
         q = self.uq(cq)
         cache, cache_t = self._views(cache)
         seq.latent_write(cols(P, "dkv"), self.dkv_norm, self.eps, sv.positions, sv.slots, self.inv_freq,
-                         self.rot_dims, cache, KR, cache_t=cache_t)
+                         self.rot_dims, cache, KR, cache_t=cache_t, **self.rot)
         qa = torch.empty(T, H, E, dtype=dt, device=dev)
         seq.gemm(q.view(T, H, D + R)[:, :, :D].permute(1, 0, 2), self.uk_t, qa[:, :, :KR].permute(1, 0, 2))
         if R:
-            seq.latent_qrope(q, sv.positions, self.inv_freq, self.rot_dims, qa, H, D, KR, R)
+            seq.latent_qrope(q, sv.positions, self.inv_freq, self.rot_dims, qa, H, D, KR, R, **self.rot)
         ol = torch.empty(T, H, KR, dtype=dt, device=dev)
         seq.latent_attn(qa, cache, sv.block_tables, sv.context_lens, sv.query_start, ol, self.scale, H, KR, R,
                         num_seqs=sv.num_seqs or None, cache_t=cache_t, window=self.window, sink=self.sink)
         og = torch.empty(T, H, V, dtype=dt, device=dev)
-        gate = cols(P, "g").unflatten(1, (H, V)).permute(1, 0, 2)
+        gate = cols(P, "g")
+        gate = (gate.unsqueeze(-1).expand(-1, -1, V) if self.head_gate else gate.unflatten(1, (H, V))).permute(1, 0, 2)
         seq.gemm(ol.permute(1, 0, 2), self.uv, og.permute(1, 0, 2), gate=gate)
         return self.o(og.view(T, H * V), out_f32=self.out_f32)
 
@@ -288,6 +300,8 @@ class WindowAttention:
     added to the softmax denominator), without a tensor. ``value_mix``: in every layer run with it but a step's
     first, the values become (1 - lam) v + lam v_first before they are cached, lam the tensor ``vmix`` and v_first that
     first run's values of the same token (all such layers need the same kv_heads * vdim).
+    ``keep_first`` n > 0: the first n positions of the sequence are seen beside the window. ``values`` "keys": the cached
+    values are the keys as projected (before norm and rotation); there is no value matrix and vdim = dim.
     ``maps`` {count: 2, init: d}: every head has two query / key maps (q and k carry [map 1, map 2] per head,
     each of size dim) that are two attentions over the same values; with lam = exp(lq1 . lk1) - exp(lq2 . lk2) + d
     (tensors ``lq1`` .. ``lk2`` [dim], one number per layer) the head's output is (a1 - lam a2), divided by its
@@ -311,6 +325,12 @@ class WindowAttention:
         self.chunk = int(m.get("chunk") or 0)
         if not 0 <= self.chunk <= self.FULL or (self.chunk and self.pool):
             raise ValueError("window_attention: chunk >= 1 (or none), not with pooled blocks")
+        self.keep = int(m.get("keep_first") or 0)
+        if not 0 <= self.keep <= self.FULL or (self.keep and (self.pool or self.chunk or m.get("dist_bias") or m.get("softcap"))):
+            raise ValueError("window_attention: keep_first >= 0, not with pooled blocks, chunks, a distance term or a softcap")
+        self.key_values = m.get("values") == "keys"
+        if m.get("values") not in (None, "keys") or (self.key_values and (self.V != self.D or m.get("maps") or m.get("bias"))):
+            raise ValueError("window_attention: values that are the keys need vdim = dim, one map and no biases")
         self.value_mix = bool(m.get("value_mix"))
         self.lam_v = float(tensors["vmix"].float().reshape(())) if self.value_mix else 0.0
         if self.pool and m.get("window") is None:
@@ -330,6 +350,8 @@ class WindowAttention:
         self.eps, self.f32 = eps, f32
         dev = torch.device(device)
         base = float(rot.get("base", 10000.0))
+        if seq.rope_amplitude(rot.get("scaling")) != 1.0:
+            raise ValueError("window_attention: no rotary scaling with a factor on cos and sin")
         self.inv_freq = seq.rope_inv_freq(dims, base, dev, scaling=rot.get("scaling"))
         self.v_freq = seq.rope_inv_freq(self.V, base, dev) if m.get("rotate_values") else None
         self.gated = m.get("gate") == "sigmoid"
@@ -359,7 +381,9 @@ class WindowAttention:
             dot = lambda a, b: float((tensors[a].double() * tensors[b].double()).sum())  # noqa: E731
             self.lam = math.exp(dot("lq1", "lk1")) - math.exp(dot("lq2", "lk2")) + d
             self.out_scale = 1.0 - d
-        self.in_rows = [("q", regroup(tensors["q"])), ("k", tensors["k"]), ("v", tensors["v"])]
+        self.in_rows = [("q", regroup(tensors["q"])), ("k", tensors["k"])]
+        if not self.key_values:
+            self.in_rows.append(("v", tensors["v"]))
         if self.gated:
             self.in_rows.append(("g", tensors["g"]))
         self.in_bias = {"q": regroup(tensors["q.b"]), "k": tensors["k.b"], "v": tensors["v.b"]} if m.get("bias") else {}
@@ -406,6 +430,8 @@ class WindowAttention:
         H, G, D, V = spec["heads"], spec["kv_heads"], spec["dim"], spec["vdim"]
         mp = int((spec.get("maps") or {}).get("count", 1))
         out = {"q": (H * mp * D, width), "k": (G * mp * D, width), "v": (G * V, width), "o": (width, H * V)}
+        if spec.get("values") == "keys":
+            del out["v"]
         if mp == 2:
             out.update({n: (D,) for n in ("lq1", "lk1", "lq2", "lk2")})
         if spec.get("bias"):
@@ -461,7 +487,7 @@ class WindowAttention:
         T = h.shape[0]
         kc, vc, kp, vp, vt = cache
         q = torch.empty(T, self.HQ * self.D, dtype=h.dtype, device=h.device)
-        v, v_first = cols(P, "v"), None
+        v, v_first = cols(P, "k" if self.key_values else "v"), None
         if self.value_mix:
             v_first = carry.get("values")
             if v_first is None:   # (a view of this layer's fused projection, which it keeps alive for the step)
@@ -478,7 +504,7 @@ class WindowAttention:
         seq.window_attn(q, kc, vc, kp, vp, sv.block_tables, sv.context_lens, sv.query_start, o, self.scale, self.HQ,
                         self.window, self.pool, self.sink, self.v_freq, num_seqs=sv.num_seqs or None, vt=vt,
                         bias_kind=self.bias_kind, bias_a=self.bias_a, bias_b=self.bias_b,
-                        gate=gate if self.maps == 1 else None, softcap=self.softcap, chunk=self.chunk)
+                        gate=gate if self.maps == 1 else None, softcap=self.softcap, chunk=self.chunk, keep=self.keep)
         if self.maps == 2:   # (a1 - lam a2) / rms * (1 - init) * sigmoid(gate), heads back in their own order
             both, o = o, torch.empty(T, self.H * self.V, dtype=h.dtype, device=h.device)
             seq.map_pair_combine(both, self.lam, self.out_scale, self.eps, gate, o, self.H, self.G, self.V)
@@ -645,10 +671,136 @@ class ShiftedLinearAttention:
         return self.o(out, out_f32=True)
 
 
+def _block_diagonal(a: torch.Tensor, b: torch.Tensor) -> torch.Tensor:
+    out = torch.zeros(a.shape[0] + b.shape[0], a.shape[1] + b.shape[1], dtype=a.dtype)
+    out[: a.shape[0], : a.shape[1]] = a
+    out[a.shape[0]:, a.shape[1]:] = b
+    return out
+
+
+class GatedDelta:
+    """Gated delta rule over an fp32 state [dim, vdim] per head in a state slot. spec: heads, kv_heads (query / key heads;
+    head h reads number h / (heads / kv_heads)), dim, vdim, conv (taps).
+        q, k, v = silu(short convolution of the projections);  q <- unit(q) dim^(-1/2);  k <- unit(k)
+        g = exp(-exp(A_log_h) softplus(W_a2 W_a1 h + dt_bias)) per head and key channel;  beta = sigmoid(W_b h) per head
+        S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+    Every head's o is divided by its root mean square, times ``norm`` [vdim], times sigmoid(W_g2 W_g1 h), then W_o. The
+    widths of the two low-rank pairs are the tensors'; their second matrices run as one block-diagonal product."""
+    kind = "gated_delta"
+    cache = "state"
+    UNIT_EPS = 1e-6            # unit(x) = x / sqrt(sum(x^2) + UNIT_EPS)
+
+    def __init__(self, spec: dict, width: int, eps: float, tensors: dict, device, f32: bool):
+        self.H, self.G, self.D, self.V = (int(spec[n]) for n in ("heads", "kv_heads", "dim", "vdim"))
+        self.taps = int(spec["conv"])
+        if self.G < 1 or self.H % self.G or self.D > seq.LINEAR_ATTN_MAX_DIM or self.taps < 1:
+            raise ValueError(f"gated_delta: heads a multiple of kv_heads, dim <= {seq.LINEAR_ATTN_MAX_DIM}, conv >= 1")
+        self.eps = eps
+        dev = torch.device(device)
+        if tensors["a2"].shape[1] != tensors["a1"].shape[0] or tensors["g2"].shape[1] != tensors["g1"].shape[0]:
+            raise ValueError("gated_delta: a1 / a2 or g1 / g2 disagree on their width")
+        self.in_rows = [(n, tensors[n]) for n in ("q", "k", "v", "b")] + [("ag", torch.cat([tensors["a1"], tensors["g1"]]))]
+        self.in_bias = {}
+        HV = self.H * self.V
+        self.ag2 = Proj(_block_diagonal(tensors["a2"], tensors["g2"]), dev, f32, allow_packed=False,
+                        bias=torch.cat([tensors["dt_bias"].float(), torch.zeros(HV)]))   # fp32 logits
+        self.decay = _f32(tensors["A_log"], dev).exp()
+        self.nw = _f32(tensors["norm"], dev)
+        self.conv_w = _f32(torch.cat([tensors[n + ".conv"].float() for n in ("q", "k", "v")]).t(), dev)   # [taps, channels]
+        self.o = Proj(tensors["o"], dev, f32)
+
+    @staticmethod
+    def shapes(spec: dict, width: int) -> dict:
+        H, G, D, V, taps = (spec[n] for n in ("heads", "kv_heads", "dim", "vdim", "conv"))
+        # None: the widths of the low-rank pairs, which only the checkpoint's tensors give
+        return {"q": (G * D, width), "q.conv": (G * D, taps), "k": (G * D, width), "k.conv": (G * D, taps), "v": (H * V, width),
+                "v.conv": (H * V, taps), "b": (H, width), "A_log": (H,), "norm": (V,), "a1": (None, width), "a2": (H * D, None),
+                "dt_bias": (H * D,), "g1": (None, width), "g2": (H * V, None), "o": (width, H * V)}
+
+    def allocate(self, num_blocks: int, block_size: int, num_slots: int, device) -> tuple:
+        """(the recurrence's state, the convolution's last inputs) per state slot."""
+        z = lambda *s: torch.zeros(num_slots, *s, dtype=torch.float32, device=device)  # noqa: E731
+        return z(self.H, self.D, self.V), z(self.taps - 1, self.conv_w.shape[1])
+
+    def page_bytes(self, block_size: int) -> int:
+        return 0
+
+    def nbytes(self) -> int:
+        return self.ag2.nbytes() + self.o.nbytes()
+
+    def forward(self, h, P, cols, sv, cache) -> torch.Tensor:
+        T, HD, HV = h.shape[0], self.H * self.D, self.H * self.V
+        state, conv_state = cache
+        zg = self.ag2(cols(P, "ag"), out_f32=True)
+        out = torch.empty(T, HV, dtype=h.dtype, device=h.device)
+        seq.gated_delta(cols(P, "q"), cols(P, "k"), cols(P, "v"), cols(P, "b"), zg[:, :HD], zg[:, HD:], self.decay, self.nw,
+                        self.conv_w, state, conv_state, sv.state_slots, sv.context_lens, sv.query_start, out, self.UNIT_EPS,
+                        self.D ** -0.5, self.eps, num_seqs=sv.num_seqs or None)
+        return self.o(out, out_f32=True)
+
+
+class SelectiveScan:
+    """Selective scan over an fp32 state [inner, state] in a state slot. spec: inner (channels), state, dt_rank, conv (taps).
+        [x, z] = W_in h;  x <- silu(short convolution of x + conv.b);  [r, B, C] = W_x x;  d = softplus(W_dt r + dt.b)
+        S[c, n] <- exp(-d_c exp(A_log[c, n])) S[c, n] + d_c x_c B_n;  y_c = sum_n S[c, n] C_n + D_c x_c
+    Output: W_o (y silu(z))."""
+    kind = "mamba1"
+    cache = "state"
+
+    def __init__(self, spec: dict, width: int, eps: float, tensors: dict, device, f32: bool):
+        self.C, self.N, self.R, self.taps = (int(spec[n]) for n in ("inner", "state", "dt_rank", "conv"))
+        if not 1 <= self.N <= seq.SCAN_MAX_STATES or self.taps < 1:
+            raise ValueError(f"mamba1: 1 <= state <= {seq.SCAN_MAX_STATES}, conv >= 1")
+        dev = torch.device(device)
+        self.in_rows = [("x", tensors["in"][: self.C]), ("z", tensors["in"][self.C:])]
+        self.in_bias = {}
+        w = tensors["x"]
+        if self.C % 64 == 0 and self.C >= PACKED_MIN_K and w.shape[0] % 64:   # whole 64-row tiles of the packed GEMM
+            w = torch.cat([w, torch.zeros(64 - w.shape[0] % 64, w.shape[1], dtype=w.dtype)])
+        self.x = Proj(w, dev, f32)
+        self.dt = Proj(tensors["dt"], dev, f32, allow_packed=False, bias=tensors["dt.b"])   # fp32
+        self.A = (_f32(tensors["A_log"], dev).exp() * -math.log2(math.e)).contiguous()
+        self.Dw, self.conv_b = _f32(tensors["D"], dev), _f32(tensors["conv.b"], dev)
+        self.conv_w = _f32(tensors["conv"].float().t(), dev)   # [taps, channels]
+        self.o = Proj(tensors["o"], dev, f32)
+
+    @staticmethod
+    def shapes(spec: dict, width: int) -> dict:
+        C, N, R, taps = (spec[n] for n in ("inner", "state", "dt_rank", "conv"))
+        return {"in": (2 * C, width), "conv": (C, taps), "conv.b": (C,), "x": (R + 2 * N, C), "dt": (C, R), "dt.b": (C,),
+                "A_log": (C, N), "D": (C,), "o": (width, C)}
+
+    def allocate(self, num_blocks: int, block_size: int, num_slots: int, device) -> tuple:
+        """(the scan's state, the convolution's last inputs) per state slot."""
+        z = lambda *s: torch.zeros(num_slots, *s, dtype=torch.float32, device=device)  # noqa: E731
+        return z(self.C, self.N), z(self.taps - 1, self.C)
+
+    def page_bytes(self, block_size: int) -> int:
+        return 0
+
+    def nbytes(self) -> int:
+        return self.x.nbytes() + self.dt.nbytes() + self.o.nbytes()
+
+    def forward(self, h, P, cols, sv, cache) -> torch.Tensor:
+        state, kept = cache
+        xin, z = cols(P, "x"), cols(P, "z")
+        meta = (sv.state_slots, sv.context_lens, sv.query_start)
+        x = torch.empty(h.shape[0], self.C, dtype=h.dtype, device=h.device)
+        seq.short_conv(xin, self.conv_w, self.conv_b, kept, *meta, x, num_seqs=sv.num_seqs or None)
+        p = self.x(x)
+        R, N = self.R, self.N
+        dt = self.dt(p[:, :R], out_f32=True)
+        y = torch.empty_like(x)
+        seq.selective_scan(x, dt, p[:, R: R + N], p[:, R + N: R + 2 * N], z, self.A, self.Dw, xin, state, kept, *meta, y,
+                           num_seqs=sv.num_seqs or None)
+        return self.o(y, out_f32=True)
+
+
 class ParallelMixers:
     """Two mixers side by side on the same input: y = left_scale * left(h) + right_scale * right(h).
-    spec: ``left`` / ``right`` = (key of MIXERS, that mixer's spec); tensors under ``left.`` / ``right.``.
-    ``forward`` returns the two outputs with their scales; the layer's residual kernel adds them."""
+    spec: ``left`` / ``right`` = (key of MIXERS, that mixer's spec); tensors under ``left.`` / ``right.``. ``out_norm``: each
+    output is RMS-normed over the width with the tensor ``left.out`` / ``right.out`` before it is scaled.
+    ``forward`` returns the two outputs with their scales; the layer's residual kernel norms and adds them."""
     kind = "parallel"
     cache = "both"
 
@@ -663,6 +815,7 @@ class ParallelMixers:
             self.in_bias.update({f"{side}.{n}": b for n, b in mx.in_bias.items()})
             del mx.in_rows
             self.parts.append((side, mx))
+        self.out_norms = tuple(_f32(tensors[side + ".out"], device) for side in ("left", "right")) if spec.get("out_norm") else None
 
     @staticmethod
     def shapes(spec: dict, width: int) -> dict:
@@ -670,6 +823,8 @@ class ParallelMixers:
         for side in ("left", "right"):
             kind, sub_spec = spec[side]
             out.update({f"{side}.{k}": v for k, v in MIXERS[kind].shapes(sub_spec, width).items()})
+            if spec.get("out_norm"):
+                out[side + ".out"] = (width,)
         return out
 
     def allocate(self, num_blocks: int, block_size: int, num_slots: int, device) -> tuple:
@@ -688,7 +843,7 @@ class ParallelMixers:
 
 
 MIXERS = {c.kind: c for c in (LatentAttention, GeneralDelta, WindowAttention, LinearAttention, ShiftedLinearAttention,
-                              ParallelMixers)}
+                              GatedDelta, SelectiveScan, ParallelMixers)}
 
 
 # ------------------------------------------------------------------------------------ feed-forwards

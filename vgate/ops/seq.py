@@ -1,8 +1,8 @@
 """Ops of layered hybrid models (fp32 residual stream, bf16 or fp32 activations).
 
 Same dispatch rule as the rest of :mod:`vgate.ops`: GPU tensors go to the HIP kernels
-(csrc/kernels/gemm_any.hip, seq_elementwise.hip, latent_attn.hip, delta_rule.hip) and raise if the
-extension is missing; CPU tensors run the unfused torch forms below (the CPU device of tests).
+(csrc/kernels/gemm_any.hip, seq_elementwise.hip, latent_attn.hip, delta_rule.hip, gated_delta.hip,
+selective_scan.hip, ...) and raise if the extension is missing; CPU tensors run the unfused torch forms below (the CPU device of tests).
 Everything the kernels compute in fp32 is fp32 here too; rows are rounded to the activation dtype
 at the same places.
 """
@@ -74,7 +74,7 @@ def gemm(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, w2: torch.Tensor |
          group_off: torch.Tensor | None = None, act: int = 0, limit: float = 0.0, alpha: float = 1.702) -> torch.Tensor:
     """out = epi(a @ w^T): 2-D, batched (3-D a / w / out) or grouped (2-D a / out, 3-D w, device row
     ranges ``group_off``; rows of a gathered through ``a_rows``). Epilogue: + bias, activation (pair
-    forms take ``w2``), * sigmoid(gate). fp32 accumulation; one rounding to out's dtype."""
+    forms take ``w2``), * sigmoid(gate) (a gate expanded over the columns: one per row). fp32 accumulation; one rounding to out's dtype."""
     if a.is_cuda:
         _C().gemm_any(a, w, out, w2, bias, gate, a_rows, group_off, act, limit, alpha)
         return out
@@ -158,11 +158,24 @@ def rope_inv_freq(dims: int, base: float, device, scaling: dict | None = None) -
     """f_i = base^(-2i / dims), i < dims / 2, rounded to fp32 once. ``scaling`` {factor, low, high,
     original} stretches long wavelengths (the Llama-3.1 rule): with l = 2 pi / f, f is kept where
     l < original / high, divided by factor where l > original / low, and blended linearly in
-    original / l between the two."""
+    original / l between the two. ``scaling`` {factor, fast, slow, original} is the YaRN rule: f is kept up to the
+    index whose pair turns ``fast`` times over ``original`` positions, divided by factor from the one that turns
+    ``slow`` times, and blended linearly in the index between the two (both rounded outwards to whole indices);
+    its factor on cos and sin is :func:`rope_amplitude`."""
     out = []
+    yarn = scaling is not None and "fast" in scaling
+    if yarn:
+        factor = float(scaling["factor"])
+        index = lambda turns: (dims * math.log(float(scaling["original"]) / (2.0 * math.pi * float(turns)))  # noqa: E731
+                               / (2.0 * math.log(float(base))))
+        lo = max(math.floor(index(scaling["fast"])), 0)
+        hi = min(math.ceil(index(scaling["slow"])), dims - 1)
     for i in range(dims // 2):
         f = float(base) ** (-2.0 * i / dims)
-        if scaling:
+        if yarn:
+            ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+            f = f / factor * ramp + f * (1.0 - ramp)
+        elif scaling:
             factor, low, high, orig = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
             wl = 2.0 * math.pi / f
             if wl > orig / low:
@@ -172,6 +185,11 @@ def rope_inv_freq(dims: int, base: float, device, scaling: dict | None = None) -
                 f = (1.0 - s) * f / factor + s * f
         out.append(f)
     return torch.tensor(out, dtype=torch.float32).to(device)
+
+
+def rope_amplitude(scaling: dict | None) -> float:
+    """The factor on cos and sin: 0.1 ln(factor) + 1 under YaRN scaling, else 1."""
+    return 0.1 * math.log(float(scaling["factor"])) + 1.0 if scaling and "fast" in scaling else 1.0
 
 
 def _rope_pairs(x: torch.Tensor, pos: torch.Tensor, inv_freq: torch.Tensor, dims: int) -> torch.Tensor:
@@ -203,30 +221,39 @@ def _rope_halves(x: torch.Tensor, pos: torch.Tensor, inv_freq: torch.Tensor, dim
     return y
 
 
-def latent_write(kv, w, eps, positions, slots, inv_freq, rot_dims: int, cache, rank: int, cache_t=None) -> None:
+def _latent_turn(x, positions, inv_freq, rot_dims: int, rot_half: bool, rot_amp: float) -> torch.Tensor:
+    y = (_rope_halves if rot_half else _rope_pairs)(x, positions, inv_freq, rot_dims)
+    y[..., :rot_dims] *= rot_amp
+    return y
+
+
+def latent_write(kv, w, eps, positions, slots, inv_freq, rot_dims: int, cache, rank: int, cache_t=None,
+                 rot_half: bool = False, rot_amp: float = 1.0) -> None:
     """cache[slot] = [rmsnorm(kv[:rank]) * w, rope(kv[rank:])] for every token with slot >= 0.
     ``cache_t`` (GPU, bf16): a second copy of the latent part laid out [page, column, key in page], the
-    operand layout of the MFMA attention kernel's weighted sum."""
+    operand layout of the MFMA attention kernel's weighted sum. The rotation pairs entry 2i with 2i + 1, or with
+    ``rot_half`` entry i with i + rot_dims / 2; cos and sin are multiplied by ``rot_amp``."""
     if kv.is_cuda:
-        _C().latent_write(kv, w, eps, positions, slots, inv_freq, rot_dims, cache, rank, cache_t)
+        _C().latent_write(kv, w, eps, positions, slots, inv_freq, rot_dims, cache, rank, cache_t, rot_half, rot_amp)
         return
     x = kv.float()
     c = x[:, :rank]
     c = c * (1.0 / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps)) * w
-    kr = _rope_pairs(x[:, rank:], positions, inv_freq, rot_dims)
+    kr = _latent_turn(x[:, rank:], positions, inv_freq, rot_dims, rot_half, rot_amp)
     row = torch.cat([c, kr], -1).to(cache.dtype)
     ok = slots >= 0
     cache.view(-1, cache.shape[-1])[slots[ok].long()] = row[ok]
 
 
-def latent_qrope(q, positions, inv_freq, rot_dims: int, qa, H: int, dim: int, rank: int, rot: int) -> None:
-    """qa[t, h, rank:] = rope(q[t, h, dim:])."""
+def latent_qrope(q, positions, inv_freq, rot_dims: int, qa, H: int, dim: int, rank: int, rot: int, rot_half: bool = False,
+                 rot_amp: float = 1.0) -> None:
+    """qa[t, h, rank:] = rope(q[t, h, dim:]) (``rot_half`` / ``rot_amp`` as in :func:`latent_write`)."""
     if q.is_cuda:
-        _C().latent_qrope(q, positions, inv_freq, rot_dims, qa, H, dim, rank, rot)
+        _C().latent_qrope(q, positions, inv_freq, rot_dims, qa, H, dim, rank, rot, rot_half, rot_amp)
         return
     T = q.shape[0]
     qr = q.view(T, H, dim + rot)[..., dim:].float()
-    qa.view(T, H, rank + rot)[..., rank:] = _rope_pairs(qr, positions, inv_freq, rot_dims).to(qa.dtype)
+    qa.view(T, H, rank + rot)[..., rank:] = _latent_turn(qr, positions, inv_freq, rot_dims, rot_half, rot_amp).to(qa.dtype)
 
 
 LATENT_FULL = 1 << 30   # "window" of a latent attention that sees every earlier position
@@ -447,6 +474,29 @@ def residual_norm(x: torch.Tensor, y, mult: float, w: torch.Tensor | None = None
         h_out.copy_(_normed(x[: h_out.shape[0]], eps, center) * w)
 
 
+def branch_residual(x: torch.Tensor, ys: list, eps: float, y3: torch.Tensor | None = None, outs: list | None = None) -> None:
+    """x += sum_i s_i u_i + y3 in fp32 (x fp32 [T, W]). ``ys``: up to two (y, s, w) of fp32 rows, u = y, or with a
+    weight w [W] (for both or none) u = y / sqrt(mean(y^2) + eps) * w. ``outs``: up to two (n, h): h = r * n in h's
+    dtype with r = x / sqrt(mean(x^2) + eps) of the new x."""
+    outs = outs or []
+    rows = [y for y, _, _ in ys] + ([y3] if y3 is not None else []) + [h for _, h in outs]
+    T = min(r.shape[0] for r in rows) if rows else 0
+    if x.is_cuda:
+        a = list(ys) + [(None, 1.0, None)] * (2 - len(ys))
+        o = list(outs) + [(None, None)] * (2 - len(outs))
+        _C().branch_residual(x, a[0][0], a[0][1], a[0][2], a[1][0], a[1][1], a[1][2], y3, eps, *o[0], *o[1], T)
+        return
+    for y, sc, w in ys:
+        u = y[:T].float()
+        x[:T] += sc * (u if w is None else _normed(u, eps, False) * w)
+    if y3 is not None:
+        x[:T] += y3[:T]
+    if outs:
+        r = _normed(x[:T], eps, False)
+        for n, h in outs:
+            h[:T] = (r * n).to(h.dtype)
+
+
 def pair_rows(a: torch.Tensor, b: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     """out[t] = [a[t], b[t]] (two fp32 [T, W] row sets side by side) rounded to out's dtype."""
     if a.is_cuda:
@@ -608,7 +658,7 @@ def window_pool(kc, vc, kp, vp, positions, block_tables, query_start, pool: int,
 def window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out, scale: float, H: int, window: int,
                 pool: int, sink, v_freq, num_seqs: int | None = None, vt=None, prefill_kernel: int = 0,
                 bias_kind: int = BIAS_NONE, bias_a=None, bias_b=None, gate=None, softcap: float = 0.0,
-                chunk: int = 0) -> None:
+                chunk: int = 0, keep: int = 0) -> None:
     """out[t, h] = sum_j p_j value_j over the keys position i of token t sees: the tokens j with
     0 <= i - j < window and, with ``pool`` = P > 0, the pooled row of every block b with
     b P + P - 1 <= i - window; p = softmax(scale q . key) over both kinds together, with exp(sink[h]) added
@@ -621,16 +671,18 @@ def window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out,
     1 = 16 rows per workgroup with the tiles shared out over its waves). ``softcap`` c > 0: the scaled score s
     becomes c tanh(s / c) (not together with a distance term). The value caches may have fewer heads than the key
     cache (consecutive key heads share a value head). ``chunk`` c > 0: of those keys only the ones with
-    floor(j / c) = floor(i / c) are seen (positions counted from the sequence's first; not with pooled blocks)."""
+    floor(j / c) = floor(i / c) are seen (positions counted from the sequence's first; not with pooled blocks).
+    ``keep`` n > 0: the first n positions are seen whatever the window (not with pooled blocks, chunks, a distance term
+    or a softcap)."""
     if q.is_cuda:
         parts, scratch = 1, None
         if vt is not None and WINDOW_SPLIT:   # decoded tokens of the MFMA kernel: several workgroups per 16-row tile
             parts, n = _C().window_attn_split(q.shape[0], block_tables.shape[0], H, kc.shape[1], kc.shape[3], vc.shape[3],
-                                              kc.dtype == torch.float32, kc.shape[2], chunk)
+                                              kc.dtype == torch.float32, kc.shape[2], window, chunk, keep, pool)
             if parts > 1:
                 scratch = torch.empty(n, dtype=torch.float32, device=q.device)
         _C().window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out, scale, H, window, pool, sink, v_freq, vt,
-                         prefill_kernel, bias_kind, bias_a, bias_b, gate, parts, scratch, softcap, chunk)
+                         prefill_kernel, bias_kind, bias_a, bias_b, gate, parts, scratch, softcap, chunk, keep)
         return
     G, page, D, V = kc.shape[1], kc.shape[2], kc.shape[3], vc.shape[3]
     rep = H // G
@@ -644,7 +696,8 @@ def window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out,
         for t in range(t0, t1):
             i = pos0 + t - t0
             lo = max(0, i - window + 1, i - i % chunk if chunk else 0)
-            pg, r = _seq_rows(bt, torch.arange(lo, i + 1), page)
+            seen = torch.cat([torch.arange(min(keep, lo)), torch.arange(lo, i + 1)])
+            pg, r = _seq_rows(bt, seen, page)
             K, Vv = kc[pg, :, r].float(), vc[pg, :, r].float()           # [n, G, D], [n, value heads, V]
             if Vv.shape[1] != G:
                 Vv = Vv.repeat_interleave(G // Vv.shape[1], dim=1)
@@ -659,7 +712,7 @@ def window_attn(q, kc, vc, kp, vp, block_tables, context_lens, query_start, out,
             if softcap > 0.0:
                 sc = softcap * torch.tanh(sc / softcap)
             if bias_kind != BIAS_NONE:
-                dist = (i - torch.arange(lo, i + 1))
+                dist = i - seen
                 if bias_kind == BIAS_LOG:
                     bias = -bias_a.view(H, 1) * torch.log(1.0 + bias_b.view(H, 1) * dist.float())
                 else:
@@ -744,3 +797,114 @@ def linear_attn(q, k, v, g, z, head_decay, tau: float, q_scale: float, in_silu: 
         gg = g[t0:t1].float()
         of = of * (torch.nn.functional.silu(gg) if gate_silu else torch.sigmoid(gg))
         out[t0:t1] = of.to(out.dtype)
+
+
+# ------------------------------------------------- short convolution, gated delta rule, selective scan
+def _conv_portion(x: torch.Tensor, w: torch.Tensor, b, kept: torch.Tensor | None) -> torch.Tensor:
+    """x [n, C] fp32 behind the ``kept`` [taps - 1, C] inputs before it (None: zeros), w [taps, C]; no activation."""
+    taps, n = w.shape[0], x.shape[0]
+    head = kept if kept is not None else torch.zeros(taps - 1, x.shape[1])
+    full = torch.cat([head, x])
+    y = torch.zeros_like(x) if b is None else b.expand_as(x).clone()
+    for i in range(taps):
+        y = y + w[i] * full[i: i + n]
+    return y
+
+
+def _conv_keep(x: torch.Tensor, kept: torch.Tensor | None, taps: int) -> torch.Tensor:
+    head = kept if kept is not None else torch.zeros(taps - 1, x.shape[1])
+    full = torch.cat([head, x])
+    return full[full.shape[0] - (taps - 1):].clone()
+
+
+def short_conv(x, w, b, kept, state_slots, context_lens, query_start, out, silu: bool = True, num_seqs: int | None = None) -> None:
+    """out[t, c] = act(b[c] + sum_i w[i, c] x[t - taps + 1 + i, c]) per sequence (w [taps, C] fp32, zeros before the
+    start; act: silu or none). A portion's first tokens read ``kept`` [slots, taps - 1, C] fp32, which is left alone
+    here: the op that runs the recurrence behind the convolution rewrites it."""
+    if x.is_cuda:
+        _C().short_conv(x, w, b, kept, state_slots, context_lens, query_start, out, silu)
+        return
+    for s in range(state_slots.numel() if num_seqs is None else num_seqs):
+        t0, t1, slot = int(query_start[s]), int(query_start[s + 1]), int(state_slots[s])
+        if t1 <= t0 or slot < 0:
+            continue
+        y = _conv_portion(x[t0:t1].float(), w, b, kept[slot] if int(context_lens[s]) > t1 - t0 else None)
+        out[t0:t1] = (torch.nn.functional.silu(y) if silu else y).to(out.dtype)
+
+
+def gated_delta(q, k, v, b, z, gate, decay, nw, conv_w, state, conv_state, state_slots, context_lens, query_start, out,
+                unit_eps: float, q_scale: float, eps: float, num_seqs: int | None = None, wide: int = -1) -> None:
+    """Gated delta rule over state slots, state [slots, H, D, V] fp32 (see csrc/kernels/gated_delta.hip):
+        q, k, v <- silu(short convolution);  q <- unit(q) q_scale;  k <- unit(k), unit(x) = x / sqrt(sum x^2 + unit_eps)
+        S <- diag(exp(-decay[h] softplus(z))) S;  u = sigmoid(b) (v - S^T k);  S <- S + k u^T;  o = S^T q
+        out = o / sqrt(mean(o^2) + eps) * nw * sigmoid(gate)
+    q, k [T, G D], v [T, H V] (head h reads q / k head h / (H / G)), b [T, H] in the activation dtype, z [T, H D] and
+    gate [T, H V] fp32, conv_w [taps, 2 G D + H V] fp32 (q, k, v channels), conv_state [slots, taps - 1, 2 G D + H V]: the
+    inputs before the portion, rewritten here. ``wide`` (GPU): the scan's form, -1 = by the launch's size."""
+    if q.is_cuda:
+        H, D, V = state.shape[1], state.shape[2], state.shape[3]
+        scratch = torch.empty(q.shape[0] * H * (4 * D + 2 * V), dtype=torch.float32, device=q.device)
+        _C().gated_delta(q, k, v, b, z, gate, decay, nw, conv_w, state, conv_state, state_slots, context_lens, query_start,
+                         out, unit_eps, q_scale, eps, scratch, wide)
+        return
+    H, D, V = state.shape[1], state.shape[2], state.shape[3]
+    G = q.shape[1] // D
+    act = torch.nn.functional.silu
+    unit = lambda x: x * (1.0 / torch.sqrt(x.pow(2).sum(-1, keepdim=True) + unit_eps))  # noqa: E731
+    for s in range(state_slots.numel() if num_seqs is None else num_seqs):
+        t0, t1, slot = int(query_start[s]), int(query_start[s + 1]), int(state_slots[s])
+        if t1 <= t0 or slot < 0:
+            continue
+        n = t1 - t0
+        first = int(context_lens[s]) - n <= 0
+        x = torch.cat([q[t0:t1].float(), k[t0:t1].float(), v[t0:t1].float()], -1)
+        kept = None if first else conv_state[slot]
+        y = act(_conv_portion(x, conv_w, None, kept))
+        conv_state[slot] = _conv_keep(x, kept, conv_w.shape[0])
+        rep = H // G
+        qq = (unit(y[:, : G * D].reshape(n, G, D)) * q_scale).repeat_interleave(rep, 1)
+        kk = unit(y[:, G * D: 2 * G * D].reshape(n, G, D)).repeat_interleave(rep, 1)
+        vv = y[:, 2 * G * D:].reshape(n, H, V)
+        g = torch.exp(-decay[None, :, None] * torch.nn.functional.softplus(z[t0:t1].float(), threshold=1e9).view(n, H, D))
+        beta = torch.sigmoid(b[t0:t1].float())
+        St = torch.zeros(H, D, V) if first else state[slot].clone()
+        o = torch.empty(n, H, V)
+        for i in range(n):
+            St = g[i][:, :, None] * St
+            u = beta[i][:, None] * (vv[i] - torch.einsum("hdv,hd->hv", St, kk[i]))
+            St = St + kk[i][:, :, None] * u[:, None, :]
+            o[i] = torch.einsum("hdv,hd->hv", St, qq[i])
+        state[slot] = St
+        o = (_normed(o, eps, False) * nw).reshape(n, H * V) * torch.sigmoid(gate[t0:t1])
+        out[t0:t1] = o.to(out.dtype)
+
+
+SCAN_MAX_STATES = 256   # states per channel the selective scan keeps in registers
+
+
+def selective_scan(x, dt, B, C, z, A, D, xin, state, kept, state_slots, context_lens, query_start, out,
+                   num_seqs: int | None = None) -> None:
+    """Selective scan over state slots, state [slots, channels, N] fp32 (see csrc/kernels/selective_scan.hip):
+        d = softplus(dt);  S[c, n] <- 2^(d_c A[c, n]) S[c, n] + d_c x_c B_n;  out_c = (sum_n S[c, n] C_n + D_c x_c) silu(z_c)
+    A carries the factor log2(e). ``xin`` / ``kept``: the inputs of the short convolution that made x, of which the
+    last taps - 1 are kept here."""
+    if x.is_cuda:
+        n = _C().selective_scan_scratch(x.shape[0], state_slots.numel(), state.shape[1], state.shape[2])
+        scratch = torch.empty(n, dtype=torch.float32, device=x.device)
+        _C().selective_scan(x, dt, B, C, z, A, D, xin, state, kept, state_slots, context_lens, query_start, out, scratch)
+        return
+    for s in range(state_slots.numel() if num_seqs is None else num_seqs):
+        t0, t1, slot = int(query_start[s]), int(query_start[s + 1]), int(state_slots[s])
+        if t1 <= t0 or slot < 0:
+            continue
+        first = int(context_lens[s]) - (t1 - t0) <= 0
+        St = torch.zeros_like(state[slot]) if first else state[slot].clone()
+        xx, d = x[t0:t1].float(), torch.nn.functional.softplus(dt[t0:t1].float(), threshold=1e9)
+        bb, cc = B[t0:t1].float(), C[t0:t1].float()
+        y = torch.empty_like(xx)
+        for i in range(t1 - t0):
+            St = torch.exp2(d[i][:, None] * A) * St + (d[i] * xx[i])[:, None] * bb[i][None]
+            y[i] = St @ cc[i]
+        state[slot] = St
+        kept[slot] = _conv_keep(xin[t0:t1].float(), None if first else kept[slot], kept.shape[1] + 1)
+        out[t0:t1] = ((y + D * xx) * torch.nn.functional.silu(z[t0:t1].float())).to(out.dtype)
