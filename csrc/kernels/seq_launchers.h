@@ -251,9 +251,9 @@ struct GatedDeltaArgs {
   const int32_t* context_lens = nullptr; const int32_t* query_start = nullptr;
   void* out = nullptr; int64_t ldo = 0;         // [T][H * V]
   int S = 0, H = 0, G = 0, D = 0, V = 0, f32 = 0;
-  int wide = -1;                                // scan form: 1 several columns per lane, 0 one, -1 by the launch's size
+  int wide = -1;                                // token scan with several columns per lane (1) or one (0); -1: by the launch's size, chunks if long
 };
-size_t gated_delta_scratch_floats(int T, int H, int D, int V);
+size_t gated_delta_scratch_floats(int T, int S, int H, int D, int V);
 void launch_gated_delta(const GatedDeltaArgs& a, int T, float* scratch, hipStream_t st);
 
 // Short causal convolution over time per channel and the selective scan behind it (selective_scan.hip).

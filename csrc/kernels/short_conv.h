@@ -38,12 +38,45 @@ __device__ __forceinline__ float short_conv_at(const void* x, int64_t ld, int f3
 // are read at a higher index than the one written, so ascending order is in place).
 __device__ __forceinline__ void short_conv_keep(const void* x, int64_t ld, int f32, int c, float* kept, int nk, int kc, int t0,
                                                 int t1, int pos0, int taps) {
-  for (int j = 0; j < taps - 1; ++j) {
-    const int tt = t1 - (taps - 1) + j;
-    float v = 0.f;
-    if (tt >= t0) v = conv_ldx(x, (int64_t)tt * ld + c, f32);
-    else if (pos0 > 0) v = kept[(int64_t)(tt - t0 + taps - 1) * nk + kc];
-    kept[(int64_t)j * nk + kc] = v;
+  for (int j0 = 0; j0 < taps - 1; j0 += 4) {
+    float v[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {  // four rows' loads asked for together
+      const int tt = t1 - (taps - 1) + j0 + u;
+      v[u] = 0.f;
+      if (j0 + u < taps - 1) {
+        if (tt >= t0) v[u] = conv_ldx(x, (int64_t)tt * ld + c, f32);
+        else if (pos0 > 0) v[u] = kept[(int64_t)(tt - t0 + taps - 1) * nk + kc];
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+      if (j0 + u < taps - 1) kept[(int64_t)(j0 + u) * nk + kc] = v[u];
+  }
+}
+
+// Channel c of the eight tokens from row t on, at most four taps, without activation; the rows between the tokens are
+// read once (values of rows at or past t1 mean nothing). F32: the rows' dtype.
+template <bool F32>
+__device__ __forceinline__ void short_conv_run8(const void* x, int64_t ld, int c, const float* w, int nw, int wc, const float* kept,
+                                                int nk, int kc, int t, int t0, int t1, int pos0, int taps, float (&y)[8]) {
+  float wl[4], v[11];
+#pragma unroll
+  for (int m = 0; m < 4; ++m) wl[m] = m >= 4 - taps ? w[(int64_t)max(m - (4 - taps), 0) * nw + wc] : 0.f;
+#pragma unroll
+  for (int m = 0; m < 11; ++m) v[m] = conv_ldx(x, (int64_t)min(max(t - 3 + m, t0), t1 - 1) * ld + c, F32 ? 1 : 0);
+  if (t - 3 < t0) {  // (uniform) the portion's first tokens: from the slot
+#pragma unroll
+    for (int m = 0; m < 3; ++m) {
+      const int r = t - 3 + m - t0 + taps - 1;
+      if (t - 3 + m < t0) v[m] = (pos0 > 0 && r >= 0) ? kept[(int64_t)r * nk + kc] : 0.f;
+    }
+  }
+#pragma unroll
+  for (int u = 0; u < 8; ++u) {
+    y[u] = 0.f;
+#pragma unroll
+    for (int m = 0; m < 4; ++m) y[u] = fmaf(wl[m], v[u + m], y[u]);
   }
 }
 

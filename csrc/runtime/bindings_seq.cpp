@@ -726,9 +726,9 @@ void gated_delta(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor
   p.context_lens = i32p(context_lens, "context_lens", p.S);
   p.query_start = i32p(query_start, "query_start", p.S + 1);  // values <= T: set by the step metadata
   TORCH_CHECK(scratch.is_cuda() && scratch.scalar_type() == torch::kFloat32 && scratch.is_contiguous() &&
-              (size_t)scratch.numel() >= vgate::gated_delta_scratch_floats((int)T, p.H, p.D, p.V) &&
+              (size_t)scratch.numel() >= vgate::gated_delta_scratch_floats((int)T, p.S, p.H, p.D, p.V) &&
               (reinterpret_cast<uintptr_t>(scratch.data_ptr()) & 15) == 0,
-              "gated_delta: scratch fp32 with T * H * (4 D + 2 V) elements, 16-B aligned");
+              "gated_delta: scratch fp32 with gated_delta_scratch(T, S, H, D, V) elements, 16-B aligned");
   p.wide = (int)wide;
   c10::DeviceGuard guard(q.device());
   vgate::launch_gated_delta(p, (int)T, scratch.data_ptr<float>(), cur_stream());
@@ -946,6 +946,9 @@ void bind_seq(pybind11::module& m) {
         py::arg("conv_w"), py::arg("state"), py::arg("conv_state"), py::arg("state_slots"), py::arg("context_lens"),
         py::arg("query_start"), py::arg("out"), py::arg("unit_eps"), py::arg("q_scale"), py::arg("eps"), py::arg("scratch"),
         py::arg("wide") = -1);
+  m.def("gated_delta_scratch", [](int64_t T, int64_t S, int64_t H, int64_t D, int64_t V) {
+    return (int64_t)vgate::gated_delta_scratch_floats((int)T, (int)S, (int)H, (int)D, (int)V);
+  }, "fp32 elements of scratch a gated_delta call over T rows and S sequences needs");
   m.def("short_conv", &short_conv, "short causal convolution over time per channel (+ silu) over state slots");
   m.def("selective_scan_scratch", [](int64_t T, int64_t S, int64_t C, int64_t N) {
     return (int64_t)vgate::selective_scan_scratch_floats((int)T, (int)S, (int)C, (int)N);

@@ -840,10 +840,12 @@ def gated_delta(q, k, v, b, z, gate, decay, nw, conv_w, state, conv_state, state
         out = o / sqrt(mean(o^2) + eps) * nw * sigmoid(gate)
     q, k [T, G D], v [T, H V] (head h reads q / k head h / (H / G)), b [T, H] in the activation dtype, z [T, H D] and
     gate [T, H V] fp32, conv_w [taps, 2 G D + H V] fp32 (q, k, v channels), conv_state [slots, taps - 1, 2 G D + H V]: the
-    inputs before the portion, rewritten here. ``wide`` (GPU): the scan's form, -1 = by the launch's size."""
+    inputs before the portion, rewritten here. ``wide`` (GPU): token by token with one (0) or several (1)
+    columns per lane; -1 = by the launch's size, long portions in chunks."""
     if q.is_cuda:
         H, D, V = state.shape[1], state.shape[2], state.shape[3]
-        scratch = torch.empty(q.shape[0] * H * (4 * D + 2 * V), dtype=torch.float32, device=q.device)
+        n = _C().gated_delta_scratch(q.shape[0], state_slots.numel(), H, D, V)
+        scratch = torch.empty(n, dtype=torch.float32, device=q.device)
         _C().gated_delta(q, k, v, b, z, gate, decay, nw, conv_w, state, conv_state, state_slots, context_lens, query_start,
                          out, unit_eps, q_scale, eps, scratch, wide)
         return
