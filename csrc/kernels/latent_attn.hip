@@ -28,6 +28,17 @@
 // of up to eight workgroups share such a sequence's key tiles (tile t goes to workgroup (t / 4) mod parts, wave
 // t mod 4); each leaves its merged (max, sum, weighted latent) in an fp32 scratch and latent_attn_merge_kernel
 // rescales and adds them in part order. The number of parts depends on the step's shape alone.
+// latent_attn, bf16 caches, prompt portions: tiled kernel. A workgroup owns 64 (token, head) rows and its four waves split
+// the columns instead of the rows, so that every cached element is read once per workgroup, by one wave, straight into
+// that wave's registers: wave w multiplies every fourth 32-wide piece of the query rows with the same piece of the keys
+// (partial scores of all 64 rows, summed over the waves through LDS in wave order), each wave takes the softmax of one of
+// the four row tiles, and wave w accumulates the w-th quarter of the latent for all 64 rows (P comes from LDS). A key
+// tile's fragments are asked for as soon as the ones before have been used, a phase ahead of their use; the barriers
+// (two per tile) wait for LDS traffic only. A row's running max moves only when a tile exceeds it by more than 2^8 (the
+// weights stay below 2^8 then, and the accumulators are rarely rescaled); that is decided per row, so a row's result does
+// not depend on its neighbours. The workgroups with the most keys start first.
+#include <stdlib.h>
+
 #include "common.h"
 #include "seq_launchers.h"
 
@@ -453,6 +464,167 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatentArgs a, con
   }
 }
 
+// NC: 16-column tiles of the latent per wave (rank <= 64 NC); NK: 32-wide query / key pieces per wave (E <= 128 NK).
+// E % 8 == 0 (host-checked). Pieces past the row's end and columns past the latent's last are read from clamped addresses:
+// a zero query piece or an output column that is never stored makes their value irrelevant.
+constexpr float LAZY_MAX = 8.f;
+template <int NC, int NK>
+__global__ __launch_bounds__(256) void latent_attn_tiled_kernel(LatentArgs a, const bf16_t* __restrict__ qa, int H,
+                                                                 float scale_log2e, const int32_t* __restrict__ block_tables,
+                                                                 int max_blocks, int num_pages,
+                                                                 const int32_t* __restrict__ context_lens,
+                                                                 const int32_t* __restrict__ query_start, int S,
+                                                                 const bf16_t* __restrict__ cache_t, bf16_t* __restrict__ ol,
+                                                                 int window, const float* __restrict__ sink) {
+  __shared__ __attribute__((aligned(16))) f32x4 sp[4][8][64];     // [wave][row tile, key half][lane]: partial scores
+  __shared__ __attribute__((aligned(16))) bf16_t pl[64][40];      // weights
+  __shared__ __attribute__((aligned(16))) float fac[64];          // rescaling factors, at the end 1 / row sums
+  const int E = a.rank + a.rot, KR = a.rank;
+  int s = -1, tile = 0, base = 0;
+  const int bx = gridDim.x - 1 - blockIdx.x;
+  for (int i = 0; i < S; ++i) {  // (sequence, 64-row tile) of this workgroup
+    const int nt = ((query_start[i + 1] - query_start[i]) * H + 63) / 64;
+    if (bx < base + nt) { s = i; tile = bx - base; break; }
+    base += nt;
+  }
+  if (s < 0) return;
+  const int w = threadIdx.x >> 6, l = threadIdx.x & 63, lr = l & 15, lg = l >> 4;
+  const int t0 = query_start[s], ntok = query_start[s + 1] - t0;
+  const int pos0 = context_lens[s] - ntok;
+  const int nrows = ntok * H, row0 = tile * 64;
+  const bf16_t* cache = reinterpret_cast<const bf16_t*>(a.cache);
+  bf16x8 qf[4][NK];  // A operands: lane holds Q[row 16 rt + lr][32 (w + 4 i) + 8 lg ..]
+#pragma unroll
+  for (int rt = 0; rt < 4; ++rt) {
+    const int r = row0 + 16 * rt + lr;
+    const bool ok = r < nrows;
+    const bf16_t* qrow = qa + ((int64_t)(t0 + (ok ? r / H : 0)) * H + (ok ? r % H : 0)) * E;
+#pragma unroll
+    for (int i = 0; i < NK; ++i) qf[rt][i] = frag16(qrow, 32 * (w + 4 * i) + 8 * lg, E, ok);
+  }
+  // softmax rows of this lane: row0 + 16 w + 4 lg + i; keys [lowest, limit) are visible
+  int limit[4], lowest[4];
+  float m[4], lsum[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = row0 + 16 * w + 4 * lg + i;
+    const bool ok = r < nrows;
+    limit[i] = ok ? pos0 + r / H + 1 : 0;
+    lowest[i] = max(0, limit[i] - window);
+    const bool sk = ok && sink != nullptr;
+    m[i] = sk ? sink[r % H] * 1.4426950408889634f : -INFINITY;
+    lsum[i] = (sk && lr == 0) ? 1.f : 0.f;
+  }
+  const int kmax = pos0 + min(row0 + 63, nrows - 1) / H + 1;       // workgroup-uniform
+  const int kmin = max(0, pos0 + row0 / H + 1 - window) & ~31;
+  const int32_t* bt = block_tables + (int64_t)s * max_blocks;
+  auto page_of = [&](int j) { return min(max(bt[min(j, kmax - 1) >> 4], 0), num_pages - 1); };
+  uint4 kf[2][NK], cf[NC];
+  auto load_k = [&](int p0, int p1) {
+    const bf16_t* k0 = cache + ((int64_t)p0 * 16 + lr) * E;
+    const bf16_t* k1 = cache + ((int64_t)p1 * 16 + lr) * E;
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int off = min(32 * (w + 4 * i) + 8 * lg, E - 8);
+      kf[0][i] = ld16(k0 + off);
+      kf[1][i] = ld16(k1 + off);
+    }
+  };
+  auto load_c = [&](int p0, int p1) {  // eight consecutive keys of one latent column per lane
+    const bf16_t* tp = cache_t + (int64_t)((lg >> 1) ? p1 : p0) * KR * 16 + 8 * (lg & 1);
+#pragma unroll
+    for (int c = 0; c < NC; ++c) cf[c] = ld16(tp + (int64_t)min(16 * (w * NC + c) + lr, KR - 1) * 16);
+  };
+  f32x4 O[4][NC];
+#pragma unroll
+  for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+    for (int c = 0; c < NC; ++c) O[rt][c] = f32x4{0.f, 0.f, 0.f, 0.f};
+  int p0 = page_of(kmin), p1 = page_of(kmin + 16);
+  int n0 = page_of(kmin + 32), n1 = page_of(kmin + 48);   // the next tile's pages (past the last: a page that is there)
+  load_k(p0, p1);
+  load_c(p0, p1);
+  for (int j0 = kmin; j0 < kmax; j0 += 32) {
+    f32x4 sc[4][2];
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt) sc[rt][0] = sc[rt][1] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NK; ++i)
+#pragma unroll
+      for (int rt = 0; rt < 4; ++rt) {
+        sc[rt][0] = mfma16(qf[rt][i], as_bf16x8(kf[0][i]), sc[rt][0]);
+        sc[rt][1] = mfma16(qf[rt][i], as_bf16x8(kf[1][i]), sc[rt][1]);
+      }
+    load_k(n0, n1);   // the next tile's keys: under way during the softmax and the weighted sum
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt) {
+      sp[w][2 * rt][l] = sc[rt][0];
+      sp[w][2 * rt + 1][l] = sc[rt][1];
+    }
+    lds_barrier();
+    f32x4 s0 = sp[0][2 * w][l], s1 = sp[0][2 * w + 1][l];
+#pragma unroll
+    for (int u = 1; u < 4; ++u) { s0 += sp[u][2 * w][l]; s1 += sp[u][2 * w + 1][l]; }
+    f32x4 al;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float v0 = (j0 + lr < limit[i] && j0 + lr >= lowest[i]) ? s0[i] * scale_log2e : -INFINITY;
+      const float v1 = (j0 + 16 + lr < limit[i] && j0 + 16 + lr >= lowest[i]) ? s1[i] * scale_log2e : -INFINITY;
+      const float top = group16_max(fmaxf(v0, v1));
+      const bool move = top > m[i] + LAZY_MAX;   // (m = -inf: the first visible keys; the same in the row's 16 lanes)
+      const float mo = m[i];
+      m[i] = move ? top : mo;
+      const float ms = (m[i] == -INFINITY) ? 0.f : m[i];   // a row that has seen no key yet
+      al[i] = move ? exp2f(mo - top) : 1.f;
+      const float e0 = exp2f(v0 - ms), e1 = exp2f(v1 - ms);
+      lsum[i] = lsum[i] * al[i] + e0 + e1;
+      pl[16 * w + 4 * lg + i][lr] = f2bf(e0);
+      pl[16 * w + 4 * lg + i][16 + lr] = f2bf(e1);
+    }
+    if (lr == 0) *reinterpret_cast<f32x4*>(&fac[16 * w + 4 * lg]) = al;
+    lds_barrier();
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt) {
+      const f32x4 f = *reinterpret_cast<const f32x4*>(&fac[16 * rt + 4 * lg]);
+      if (__any(f[0] != 1.f || f[1] != 1.f || f[2] != 1.f || f[3] != 1.f)) {
+#pragma unroll
+        for (int c = 0; c < NC; ++c) O[rt][c] *= f;
+      }
+      const bf16x8 pf = as_bf16x8(*reinterpret_cast<const uint4*>(&pl[16 * rt + lr][8 * lg]));
+#pragma unroll
+      for (int c = 0; c < NC; ++c) O[rt][c] = mfma16(pf, as_bf16x8(cf[c]), O[rt][c]);
+    }
+    load_c(n0, n1);
+    __builtin_amdgcn_sched_barrier(0);
+    n0 = page_of(j0 + 64);
+    n1 = page_of(j0 + 80);
+  }
+  {
+    f32x4 inv;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) inv[i] = 1.f / group16_sum(lsum[i]);
+    __syncthreads();   // every wave has read the last tile's factors
+    if (lr == 0) *reinterpret_cast<f32x4*>(&fac[16 * w + 4 * lg]) = inv;
+    __syncthreads();
+  }
+#pragma unroll
+  for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int rl = 16 * rt + 4 * lg + i, r = row0 + rl;
+      if (r < nrows) {
+        const float inv = fac[rl];
+        bf16_t* orow = ol + ((int64_t)(t0 + r / H) * H + r % H) * KR;
+#pragma unroll
+        for (int c = 0; c < NC; ++c) {
+          const int col = 16 * (w * NC + c) + lr;
+          if (col < KR) orow[col] = f2bf(O[rt][c][i] * inv);
+        }
+      }
+    }
+}
+
 // The rows of a split sequence from the partial results of `parts` workgroups: M = max of the parts' maxima (log2
 // units), sums and weighted latents rescaled by 2^(M_p - M) and added in part order, then normalised and stored.
 // vs: the row stride of the parts' weighted latents.
@@ -494,11 +666,27 @@ __global__ __launch_bounds__(256) void latent_attn_merge_kernel(int rank, int H,
   }
 }
 
+// VGATE_LATENT_TILED=0: prompt portions on the kernel whose waves split the rows
+bool tiled_prefill() {
+  static const bool on = [] {
+    const char* e = getenv("VGATE_LATENT_TILED");
+    return e == nullptr || e[0] != '0';
+  }();
+  return on;
+}
+
 template <int NCT, int NQF>
 void launch_mfma(const LatentArgs& a, const void* qa, int H, float scale, const int32_t* block_tables, int max_blocks,
                  int num_pages, const int32_t* context_lens, const int32_t* query_start, int S, const void* cache_t,
                  void* ol, int window, const float* sink, int parts, float* scratch, hipStream_t st) {
   const int blocks = (a.T * H + 63) / 64 + S;
+  if ((int64_t)a.T * H > 16 * (int64_t)S && tiled_prefill()) {  // (prompt portions among the step's sequences)
+    hipLaunchKernelGGL((latent_attn_tiled_kernel<NCT / 4, (NQF + 3) / 4>), dim3(blocks), dim3(256), 0, st, a,
+                       reinterpret_cast<const bf16_t*>(qa), H, scale * 1.4426950408889634f, block_tables, max_blocks, num_pages,
+                       context_lens, query_start, S, reinterpret_cast<const bf16_t*>(cache_t), reinterpret_cast<bf16_t*>(ol),
+                       window, sink);
+    return;
+  }
   float* part_o = scratch;
   float* part_ml = parts > 1 ? scratch + (size_t)parts * blocks * 16 * 16 * NCT : nullptr;
   hipLaunchKernelGGL((latent_attn_mfma_kernel<NCT, NQF>), dim3(blocks, parts), dim3(256), 0, st, a,
