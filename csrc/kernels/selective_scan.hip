@@ -7,8 +7,8 @@
 //   short_conv   one thread per (token, eight channels): convolution, bias, silu (scalar form for other alignments).
 //   scan         lane = (channel, one of LPC parts of its states), NS states in registers; per token and state one exp2,
 //                two FMAs and a product, LPC lanes meet in log2(LPC) lane exchanges. Tokens are staged through LDS TC at
-//                a time (softplus taken there) while the next TC load into registers; y leaves through LDS so that the
-//                gate, D x and the store run over whole rows of channels.
+//                a time (softplus, D x and the gate taken there) while the next TC load into registers; outputs leave through
+//                LDS, so that the stores run over whole rows of channels. One barrier per TC tokens.
 // Long steps run the scan over chunks of CH tokens in parallel:
 //   local   every chunk from a zero state: its local state L_c and its sum of steps s_c
 //   carry   per sequence, chunk after chunk: I_0 = slot state, I_(c+1) = exp(s_c A) I_c + L_c (the same recurrence taken
@@ -100,13 +100,15 @@ __device__ __forceinline__ bool locate_chunk(const SelectiveScanArgs& p, int CH,
 
 // MODE WHOLE: blockIdx.x a sequence, its whole portion from its slot. LOCAL / OUTPUT: blockIdx.x one chunk of CH tokens
 // (chunks of all sequences numbered in order). blockIdx.y: 256 / LPC channels.
-template <int LPC, int NS, int MODE>
+template <int LPC, int NS, int MODE, bool F32>
 __global__ __launch_bounds__(256) void selective_scan_kernel(SelectiveScanArgs p, int CH, float* __restrict__ cstate,
                                                               float* __restrict__ cstep) {
   constexpr int TC = 8, CPB = 256 / LPC, NT = LPC * NS;
   constexpr int NX = (TC * CPB + 255) / 256, NB = (TC * NT + 255) / 256;
-  __shared__ __attribute__((aligned(16))) float lb[2][TC][NT], lc[2][TC][NT];
-  __shared__ float ld[2][TC][CPB], lx[2][TC][CPB], ly[TC][CPB];
+  constexpr bool OUT = MODE != SCAN_LOCAL;
+  __shared__ __attribute__((aligned(16))) float lb[2][TC][NT], lc[OUT ? 2 : 1][TC][NT];
+  __shared__ __attribute__((aligned(16))) float4 lt[2][TC][CPB];   // {d, d x, D x, silu(z)} of a token and channel
+  __shared__ float ly[OUT ? 2 : 1][TC][CPB];
   int s = blockIdx.x, t0, t1;
   if (MODE == SCAN_WHOLE) {
     t0 = p.query_start[s]; t1 = p.query_start[s + 1];
@@ -128,21 +130,32 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelectiveScanArgs p
     A[j] = on ? ap[j] : 0.f;
     S[j] = (on && !from_zero) ? sp[j] : 0.f;
   }
-  float pd[NX], px[NX], pb[NB], pc[NB];
+  float Dc[NX], pd[NX], px[NX], pz[NX], pb[NB], pc[NB];
+#pragma unroll
+  for (int r = 0; r < NX; ++r) {
+    const int cc = cb + (tid + 256 * r) % CPB;
+    Dc[r] = (OUT && cc < C) ? p.D[cc] : 0.f;
+  }
+  // rows past the portion's end and channels past the last are read from clamped places (their results are never used);
+  // states past the last have B = C = 0
+  constexpr int RX = 256 / CPB;   // tokens apart of a thread's pieces
+  const int xcol = min(cb + tid % CPB, C - 1);
+  const int row = tid / CPB;
   auto fetch = [&](int tb) {
 #pragma unroll
     for (int r = 0; r < NX; ++r) {
-      const int e = tid + 256 * r, t = tb + e / CPB, cc = cb + e % CPB;
-      const bool ok = e < TC * CPB && t < t1 && cc < C;
-      pd[r] = ok ? p.dt[(int64_t)t * p.lddt + cc] : 0.f;
-      px[r] = ok ? conv_ldx(p.x, (int64_t)t * p.ldx + cc, p.f32) : 0.f;
+      const int t = min(tb + row + RX * r, t1 - 1);
+      pd[r] = p.dt[(int64_t)t * p.lddt + xcol];
+      px[r] = conv_ldx(p.x, (int64_t)t * p.ldx + xcol, F32 ? 1 : 0);
+      if (OUT) pz[r] = conv_ldx(p.z, (int64_t)t * p.ldz + xcol, F32 ? 1 : 0);
     }
 #pragma unroll
     for (int r = 0; r < NB; ++r) {
-      const int e = tid + 256 * r, t = tb + e / NT, n = e % NT;
-      const bool ok = e < TC * NT && t < t1 && n < N;
-      pb[r] = ok ? conv_ldx(p.B, (int64_t)t * p.ldbc + n, p.f32) : 0.f;
-      pc[r] = (ok && MODE != SCAN_LOCAL) ? conv_ldx(p.Cm, (int64_t)t * p.ldbc + n, p.f32) : 0.f;
+      const int e = tid + 256 * r, n = e % NT;
+      const int64_t o = (int64_t)min(tb + e / NT, t1 - 1) * p.ldbc + min(n, N - 1);
+      pb[r] = conv_ldx(p.B, o, F32 ? 1 : 0);
+      if (OUT) pc[r] = conv_ldx(p.Cm, o, F32 ? 1 : 0);
+      if (n >= N) pb[r] = pc[r] = 0.f;
     }
   };
   auto put = [&](int buf) {
@@ -151,56 +164,57 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(SelectiveScanArgs p
       const int e = tid + 256 * r;
       if (e < TC * CPB) {
         const float d = softplus_f(pd[r]);
-        (&ld[buf][0][0])[e] = d;
-        (&lx[buf][0][0])[e] = d * px[r];
+        (&lt[buf][0][0])[e] = make_float4(d, d * px[r], OUT ? Dc[r] * px[r] : 0.f, OUT ? silu_f(pz[r]) : 0.f);
       }
     }
 #pragma unroll
     for (int r = 0; r < NB; ++r) {
       const int e = tid + 256 * r;
-      if (e < TC * NT) { (&lb[buf][0][0])[e] = pb[r]; (&lc[buf][0][0])[e] = pc[r]; }
+      if (e < TC * NT) {
+        (&lb[buf][0][0])[e] = pb[r];
+        if (OUT) (&lc[OUT ? buf : 0][0][0])[e] = pc[r];
+      }
+    }
+  };
+  auto store = [&](int tb, int nt, int buf) {  // a finished tile's rows of channels
+    for (int e = tid; e < nt * CPB; e += 256) {
+      const int cc = cb + e % CPB;
+      if (cc >= C) continue;
+      const float o = (&ly[OUT ? buf : 0][0][0])[e];
+      const int64_t oi = (int64_t)(tb + e / CPB) * p.ldo + cc;
+      if (F32) reinterpret_cast<float*>(p.out)[oi] = o;
+      else reinterpret_cast<bf16_t*>(p.out)[oi] = f2bf(o);
     }
   };
   fetch(t0);
   put(0);
-  __syncthreads();
+  lds_barrier();
   int buf = 0;
   for (int tb = t0; tb < t1; tb += TC) {
     const bool more = tb + TC < t1;
     if (more) fetch(tb + TC);
+    if (OUT && tb > t0) store(tb - TC, TC, buf ^ 1);
     const int nt = min(TC, t1 - tb);
 #pragma unroll
     for (int i = 0; i < TC; ++i) {
       if (i >= nt) break;
-      const float d = ld[buf][i][cl], dx = lx[buf][i][cl];
+      const float4 x = lt[buf][i][cl];
       float y = 0.f;
 #pragma unroll
       for (int j = 0; j < NS; ++j) {
-        S[j] = fmaf(__builtin_amdgcn_exp2f(d * A[j]), S[j], dx * lb[buf][i][n0 + j]);
-        if (MODE != SCAN_LOCAL) y = fmaf(S[j], lc[buf][i][n0 + j], y);
+        S[j] = fmaf(__builtin_amdgcn_exp2f(x.x * A[j]), S[j], x.y * lb[buf][i][n0 + j]);
+        if (OUT) y = fmaf(S[j], lc[OUT ? buf : 0][i][n0 + j], y);
       }
-      if (MODE == SCAN_LOCAL) {
-        steps += d;
-      } else {
+      if (OUT) {
         y = part_sum<LPC>(y);
-        if (part == 0) ly[i][cl] = y;
+        if (part == 0) ly[OUT ? buf : 0][i][cl] = (y + x.z) * x.w;
+      } else {
+        steps += x.x;
       }
     }
-    if (MODE != SCAN_LOCAL) {
-      __syncthreads();
-      for (int e = tid; e < nt * CPB; e += 256) {
-        const int t = tb + e / CPB, cc = cb + e % CPB;
-        if (cc < C) {
-          const float xv = conv_ldx(p.x, (int64_t)t * p.ldx + cc, p.f32);
-          const float o = fmaf(p.D[cc], xv, (&ly[0][0])[e]) * silu_f(conv_ldx(p.z, (int64_t)t * p.ldz + cc, p.f32));
-          const int64_t oi = (int64_t)t * p.ldo + cc;
-          if (p.f32) reinterpret_cast<float*>(p.out)[oi] = o;
-          else reinterpret_cast<bf16_t*>(p.out)[oi] = f2bf(o);
-        }
-      }
-    }
-    if (more) put(buf ^ 1);  // (the other buffer: every wave left it at the barrier before this tile)
-    __syncthreads();         // (also: ly is rewritten by the next tile)
+    if (more) put(buf ^ 1);  // (every wave left that buffer before the last barrier)
+    lds_barrier();
+    if (!more && OUT) store(tb, nt, buf);
     buf ^= 1;
   }
   if (MODE == SCAN_OUTPUT) return;
@@ -248,19 +262,24 @@ __global__ __launch_bounds__(256) void selective_carry_kernel(SelectiveScanArgs 
   }
 }
 
-template <int LPC, int NS>
-void launch_scan(const SelectiveScanArgs& a, int T, float* cstate, float* cstep, hipStream_t st) {
+template <int LPC, int NS, bool F32>
+void launch_scan_as(const SelectiveScanArgs& a, int T, float* cstate, float* cstep, hipStream_t st) {
   constexpr int CPB = 256 / LPC;
   const int CH = selective_scan_chunk_size(T, a.S), cols = (a.C + CPB - 1) / CPB;
   if (CH <= 0) {
-    hipLaunchKernelGGL((selective_scan_kernel<LPC, NS, SCAN_WHOLE>), dim3(a.S, cols), dim3(256), 0, st, a, 0, nullptr, nullptr);
+    hipLaunchKernelGGL((selective_scan_kernel<LPC, NS, SCAN_WHOLE, F32>), dim3(a.S, cols), dim3(256), 0, st, a, 0, nullptr, nullptr);
     return;
   }
   const int chunks = T / CH + a.S;
-  hipLaunchKernelGGL((selective_scan_kernel<LPC, NS, SCAN_LOCAL>), dim3(chunks, cols), dim3(256), 0, st, a, CH, cstate, cstep);
+  hipLaunchKernelGGL((selective_scan_kernel<LPC, NS, SCAN_LOCAL, F32>), dim3(chunks, cols), dim3(256), 0, st, a, CH, cstate, cstep);
   const int64_t ey = ((int64_t)a.C * a.N + 255) / 256;
   hipLaunchKernelGGL(selective_carry_kernel, dim3(a.S, (unsigned)(ey < 1024 ? ey : 1024)), dim3(256), 0, st, a, CH, cstate, cstep);
-  hipLaunchKernelGGL((selective_scan_kernel<LPC, NS, SCAN_OUTPUT>), dim3(chunks, cols), dim3(256), 0, st, a, CH, cstate, cstep);
+  hipLaunchKernelGGL((selective_scan_kernel<LPC, NS, SCAN_OUTPUT, F32>), dim3(chunks, cols), dim3(256), 0, st, a, CH, cstate, cstep);
+}
+template <int LPC, int NS>
+void launch_scan(const SelectiveScanArgs& a, int T, float* cstate, float* cstep, hipStream_t st) {
+  if (a.f32) launch_scan_as<LPC, NS, true>(a, T, cstate, cstep, st);
+  else launch_scan_as<LPC, NS, false>(a, T, cstate, cstep, st);
 }
 
 }  // namespace
