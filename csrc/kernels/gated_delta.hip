@@ -277,13 +277,20 @@ __device__ __forceinline__ float row_dot(const float* row, const float (&x)[CN],
   return a + b;
 }
 
-// grid (chunk, head)
+// first float of row i of a packed lower triangle whose row i has i entries, padded to whole 16-B pieces (row i of one with
+// the diagonal: tri(i + 1))
+__host__ __device__ constexpr int tri(int i) {
+  const int n = i > 0 ? i - 1 : 0, g = n / 4;
+  return i > 0 ? 4 * (2 * g * (g + 1) + (n - 4 * g) * (g + 1)) : 0;
+}
+
+// grid (chunk, head). At DP = 128 the LDS comes to a third of a CU's.
 template <int DP, bool F32>
-__global__ __launch_bounds__(256) void gated_delta_chunk_kernel(GatedDeltaArgs p, float* __restrict__ rec) {
+__global__ __launch_bounds__(256, DP > 64 ? 3 : 4) void gated_delta_chunk_kernel(GatedDeltaArgs p, float* __restrict__ rec) {
   constexpr int X = DP / 32;   // 16-B pieces of a row a lane of the pair sums holds: channels 32 x + 4 dg ..
   __shared__ __attribute__((aligned(16))) float lk[CN][DP], lq[CN][DP], lg[CN][DP];
-  __shared__ __attribute__((aligned(16))) float As[CN][CN + 4], Bs[CN][CN + 4];
-  __shared__ float rn[2 * CN], beta[CN];   // 1 / norms of q (times q_scale), then of k
+  __shared__ __attribute__((aligned(16))) float As[tri(CN)], Bs[tri(CN + 1)];
+  __shared__ float beta[CN];
   int s, t0, t1;
   if (!locate_chunk(p, blockIdx.x, s, t0, t1)) return;
   const int h = blockIdx.y, D = p.D, V = p.V, H = p.H, GD = p.G * D;
@@ -315,30 +322,35 @@ __global__ __launch_bounds__(256) void gated_delta_chunk_kernel(GatedDeltaArgs p
   }
   if (tid < CN) beta[tid] = t0 + tid < t1 ? sigm(conv_ldx(p.b, (int64_t)(t0 + tid) * p.ldb + h, F32 ? 1 : 0)) : 0.f;
   __syncthreads();
-  {  // four threads per row
+  {  // unit norms of q (times q_scale) and k in place: four threads per row
     const int row = tid >> 2, part = tid & 3;
-    const float* x = row < CN ? lq[row] : lk[row - CN];
+    float* x = row < CN ? lq[row] : lk[row - CN];
+    float4 v[DP / 16];
     float ss = 0.f;
 #pragma unroll
     for (int m = 0; m < DP / 16; ++m) {
-      const float4 v = *reinterpret_cast<const float4*>(x + 16 * m + 4 * part);
-      ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+      v[m] = *reinterpret_cast<const float4*>(x + 16 * m + 4 * part);
+      ss = fmaf(v[m].x, v[m].x, fmaf(v[m].y, v[m].y, fmaf(v[m].z, v[m].z, fmaf(v[m].w, v[m].w, ss))));
     }
     ss += row_rot<0xB1>(ss);   // (quad_perm [1, 0, 3, 2], then [2, 3, 0, 1])
     ss += row_rot<0x4E>(ss);
-    if (part == 0) rn[row] = 1.f / sqrtf(ss + p.unit_eps) * (row < CN ? p.q_scale : 1.f);
+    const float f = 1.f / sqrtf(ss + p.unit_eps) * (row < CN ? p.q_scale : 1.f);
+#pragma unroll
+    for (int m = 0; m < DP / 16; ++m)
+      *reinterpret_cast<float4*>(x + 16 * m + 4 * part) = make_float4(v[m].x * f, v[m].y * f, v[m].z * f, v[m].w * f);
   }
   __syncthreads();
-  {  // a and b: wave wv owns the columns j = 8 wv .., lane = (channel group dg of eight, j)
-    const int dg = lane >> 3, j = 8 * wv + (lane & 7);
+  {  // a and b: a wave owns eight columns j, lane = (channel group dg of eight, j); the wave with most rows differs
+     // between neighbouring chunks, so that workgroups on one CU do not all load the same SIMD
+    const int jb = (blockIdx.x & 1) ? 3 - wv : wv;
+    const int dg = lane >> 3, j = 8 * jb + (lane & 7);
     float r[4 * X];
-    const float kn = rn[CN + j];
 #pragma unroll
     for (int x = 0; x < X; ++x) {
       const float4 v = *reinterpret_cast<const float4*>(&lk[j][32 * x + 4 * dg]);
-      r[4 * x] = v.x * kn; r[4 * x + 1] = v.y * kn; r[4 * x + 2] = v.z * kn; r[4 * x + 3] = v.w * kn;
+      r[4 * x] = v.x; r[4 * x + 1] = v.y; r[4 * x + 2] = v.z; r[4 * x + 3] = v.w;
     }
-    for (int i = 8 * wv; i < CN; ++i) {
+    for (int i = 8 * jb; i < CN; ++i) {
       float a = 0.f, b = 0.f;
 #pragma unroll
       for (int x = 0; x < X; ++x) {
@@ -351,7 +363,8 @@ __global__ __launch_bounds__(256) void gated_delta_chunk_kernel(GatedDeltaArgs p
       }
       a = key_sum<8>(a);
       b = key_sum<8>(b);
-      if (dg == 0) { As[i][j] = a * rn[CN + i]; Bs[i][j] = b * rn[i]; }   // (i < j, and a at i = j: never used)
+      if (dg == 0 && i > j) As[tri(i) + j] = a;
+      if (dg == 0 && i >= j) Bs[tri(i + 1) + j] = b;
     }
   }
   __syncthreads();
@@ -362,7 +375,7 @@ __global__ __launch_bounds__(256) void gated_delta_chunk_kernel(GatedDeltaArgs p
 #pragma unroll
       for (int i = 0; i < CN; ++i) {
         gm *= lg[i][c];
-        x[i] = gm * lk[i][c] * rn[CN + i];
+        x[i] = gm * lk[i][c];
       }
     } else {
       const int vc = h * V + c - D, col = 2 * GD + vc;
@@ -375,7 +388,10 @@ __global__ __launch_bounds__(256) void gated_delta_chunk_kernel(GatedDeltaArgs p
       }
     }
 #pragma unroll
-    for (int i = 0; i < CN; ++i) x[i] = beta[i] * (x[i] - row_dot(As[i], x, i));
+    for (int i = 0; i < CN; ++i) {
+      x[i] = beta[i] * (x[i] - row_dot(As + tri(i), x, i));
+      if (i % 2) __builtin_amdgcn_sched_barrier(0);   // (rows ahead of time would take hundreds of registers)
+    }
     if (c < D) {
       float gb = 1.f;
 #pragma unroll
@@ -383,10 +399,11 @@ __global__ __launch_bounds__(256) void gated_delta_chunk_kernel(GatedDeltaArgs p
         f32x4 v;
 #pragma unroll
         for (int j = 3; j >= 0; --j) {
-          v[j] = lk[j0 + j][c] * rn[CN + j0 + j] * gb;
+          v[j] = lk[j0 + j][c] * gb;
           gb *= lg[j0 + j][c];
         }
         *reinterpret_cast<f32x4*>(kt + c * CN + j0) = v;
+        __builtin_amdgcn_sched_barrier(0);
       }
       gam[c] = gb;
       float gm = 1.f;
@@ -394,16 +411,18 @@ __global__ __launch_bounds__(256) void gated_delta_chunk_kernel(GatedDeltaArgs p
       for (int i = 0; i < CN; ++i) {
         gm *= lg[i][c];
         r0[i * DP + c] = x[i];
-        r0[(CN + i) * DP + c] = gm * lq[i][c] * rn[i] - row_dot(Bs[i], x, i + 1);
+        r0[(CN + i) * DP + c] = gm * lq[i][c] - row_dot(Bs + tri(i + 1), x, i + 1);
+        if (i % 2) __builtin_amdgcn_sched_barrier(0);
       }
     } else {
 #pragma unroll
       for (int i0 = 0; i0 < CN; i0 += 4) {
         f32x4 v;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = row_dot(Bs[i0 + i], x, i0 + i + 1);
+        for (int i = 0; i < 4; ++i) v[i] = row_dot(Bs + tri(i0 + i + 1), x, i0 + i + 1);
         *reinterpret_cast<f32x4*>(vh + (c - D) * CN + i0) = f32x4{x[i0], x[i0 + 1], x[i0 + 2], x[i0 + 3]};
         *reinterpret_cast<f32x4*>(cc + (c - D) * CN + i0) = v;
+        __builtin_amdgcn_sched_barrier(0);
       }
     }
   }
