@@ -721,16 +721,21 @@ def test_selective_scan_alone(device, C, N, taps):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("C", [24, 520])
-def test_short_conv_bf16_vector_form(C):
-    """bf16 rows in 16-B pieces (a column view of a wider projection) against the scalar form of an odd view."""
+@pytest.mark.parametrize("taps", [1, 2, 4, 6])
+@pytest.mark.parametrize("lens", [[8, 13], [2, 300, 1, 8, 7, 266]])
+def test_short_conv_bf16_vector_forms(C, taps, lens):
+    """bf16 rows in 16-B pieces (a column view of a wider projection) against the scalar form of an odd view and the plain
+    form; sequences that start and go on, longer and shorter than the taps."""
     from vgate.ops import seq
     d = torch.device("cuda")
     g = torch.Generator().manual_seed(3)
-    T, taps = 21, 4
+    T, S = sum(lens), len(lens)
     P = torch.randn(T, 2 * C, generator=g).to(d, torch.bfloat16)
-    w, b, kept = torch.randn(taps, C, generator=g).to(d), torch.randn(C, generator=g).to(d), torch.randn(2, taps - 1, C, generator=g).to(d)
+    w, b, kept = torch.randn(taps, C, generator=g).to(d), torch.randn(C, generator=g).to(d), torch.randn(S, taps - 1, C, generator=g).to(d)
     i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=d)  # noqa: E731
-    slots, cl, qs = i32([1, 0]), i32([8 + 13, 13]), i32([0, 8, 21])   # the first sequence goes on at position 13
+    slots = i32(list(reversed(range(S))))
+    cl = i32([n + (13 if s % 2 == 0 else 0) for s, n in enumerate(lens)])    # every other sequence goes on at position 13
+    qs = i32([sum(lens[:s]) for s in range(S + 1)])
     a, o = torch.zeros(T, C, dtype=torch.bfloat16, device=d), torch.zeros(T, C + 1, dtype=torch.bfloat16, device=d)[:, 1:]
     seq.short_conv(P[:, C:], w, b, kept, slots, cl, qs, a)
     seq.short_conv(P[:, C:], w, b, kept, slots, cl, qs, o)
